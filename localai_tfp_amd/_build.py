@@ -32,6 +32,7 @@ BUILD = ROOT / "build" / "native"
 ARCH = os.environ.get("MX_OFFLOAD_ARCH", "gfx950")
 HIPCC = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
 CXX = os.environ.get("CXX", "g++")
+NO_PACKED_FP32 = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
 
 
 def _hash(paths):
@@ -137,6 +138,9 @@ def build_kernels(verbose=False) -> Path:
         "-std=c++17",
         "-munsafe-fp-atomics",
         "-ffp-contract=fast",
+        # no packed fp32 instructions: some of their forms have given wrong results (the host pass warns that it does
+        # not know the feature, which is harmless)
+        *NO_PACKED_FP32,
         "-I",
         str(kdir),
         "-Wno-unused-result",
@@ -151,7 +155,7 @@ def build_latent(verbose=False) -> Path:
     srcs = sorted((kdir / "latent").glob("*.hip"))
     headers = sorted(kdir.glob("*.h"))
     cflags = [f"--offload-arch={ARCH}", "-O3", "-fPIC", "-std=c++17", "-ffp-contract=fast",
-              "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops", "-I", str(kdir), "-Wno-unused-result",
+              *NO_PACKED_FP32, "-I", str(kdir), "-Wno-unused-result",
               "-Wno-unknown-warning-option"]
     return _build_lib("libmxl.so", srcs, headers, HIPCC, cflags, ["-fPIC"], verbose)
 
@@ -163,7 +167,7 @@ def build_hybrid(verbose=False) -> Path:
     srcs = sorted((kdir / "hybrid").glob("*.hip"))
     headers = sorted(kdir.glob("*.h"))
     cflags = [f"--offload-arch={ARCH}", "-O3", "-fPIC", "-std=c++17", "-ffp-contract=fast",
-              "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops", "-I", str(kdir), "-Wno-unused-result",
+              *NO_PACKED_FP32, "-I", str(kdir), "-Wno-unused-result",
               "-Wno-unknown-warning-option"]
     return _build_lib("libmxh.so", srcs, headers, HIPCC, cflags, ["-fPIC"], verbose)
 
