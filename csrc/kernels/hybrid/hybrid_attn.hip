@@ -4,7 +4,8 @@
 // The value pool may hold fewer heads than the key pool (gv of them, a divisor of G): key head g then reads value head
 // g % gv, several attention maps over the same values. Every kernel also takes an AttnExtra: a learned sink score per
 // head instead of 0, an additive bias looked up by the distance between query and key (table [H, distances], the last
-// entry serving every larger distance), and a gate per row and head whose sigmoid multiplies the head's output.
+// entry serving every larger distance), a gate per row and head whose sigmoid multiplies the head's output, and a count
+// of first tokens (`keep`) that stay visible in front of a window.
 //
 // attn_rows_kernel: one wave per (query row, query head). Keys are taken 64 at a time, one per lane: the lane forms
 // its key's whole score against the query (held in LDS as fp32, pre-multiplied by the scale), the wave updates the
@@ -33,7 +34,18 @@ struct AttnExtra {
     const float* gate;    // pre-sigmoid gate of row r and head h at gate[r * ldg + h] (null: none)
     int ldg;
     int gv;               // value heads in the pool: key head g reads value head g % gv
+    int keep;             // with a window: positions 0 .. keep - 1 stay visible whatever their distance
 };
+// Visible keys of a row whose window starts at lo: the kept first tokens [0, kn) that lie in front of it, then [lo, pos].
+// The kernels that serve one position per wave count them as one range: visible key v is at position v < kn ? v : v + gap.
+struct KeyRange {
+    int kn, gap;
+    MX_DEV int pos(int v) const { return v < kn ? v : v + gap; }
+};
+MX_DEV KeyRange key_range(int lo, int window, int keep) {
+    const int kn = window > 0 ? min(keep, lo) : 0;
+    return {kn, lo - kn};
+}
 MX_DEV float sink_score(const AttnExtra& ex, int h) { return ex.sink_v ? ex.sink_v[h] : 0.f; }
 MX_DEV float dist_bias(const AttnExtra& ex, int dist, int H, int h) {
     return ex.bias[(long)h * ex.nb + min(max(dist, 0), ex.nb - 1)];
@@ -153,11 +165,13 @@ __global__ __launch_bounds__(64) void attn_rows_kernel(const void* q, int ldq, c
     const int g = h0 / (H / G);
     const long qrow = (long)(row_base + r) * ldq + (long)h0 * dk;
     for (int e = lane; e < REP * dk; e += 64) qs[e] = ld1<B16>(q, qrow + e) * scale;
-    int lo = chunk > 0 ? (pos / chunk) * chunk : window > 0 ? max(0, pos - window + 1) : 0;
+    const int lo = chunk > 0 ? (pos / chunk) * chunk : window > 0 ? max(0, pos - window + 1) : 0;
     const int qpos = pos;
+    const KeyRange kr = key_range(lo, window, ex.keep);
+    int v_begin = 0, v_end = pos + 1 - kr.gap;  // visible keys [v_begin, v_end)
     if (parts > 1) {  // this partition's keys; the sink joins in the merge
-        lo += z * part_len;
-        pos = min(pos, lo + part_len - 1);
+        v_begin = z * part_len;
+        v_end = min(v_end, v_begin + part_len);
         sink = 0;
     }
     const int* table = bt + (long)s * bt_stride;
@@ -170,9 +184,9 @@ __global__ __launch_bounds__(64) void attn_rows_kernel(const void* q, int ldq, c
         for (int u = 0; u < DVU; ++u) acc[i][u] = 0.f;
     }
     __syncthreads();
-    for (int j0 = lo; j0 <= pos; j0 += 64) {
-        const int j = j0 + lane;
-        const bool ok = j <= pos;
+    for (int j0 = v_begin; j0 < v_end; j0 += 64) {
+        const bool ok = j0 + lane < v_end;
+        const int j = kr.pos(j0 + lane);
         float sc[REP];
         long tok = 0;
         if (ok) {
@@ -189,7 +203,7 @@ __global__ __launch_bounds__(64) void attn_rows_kernel(const void* q, int ldq, c
             const float si = ok ? sc[i] : -INFINITY;
             const float mn = fmaxf(m[i], wave_max(si));
             p[i] = ok ? expf(si - mn) : 0.f;
-            alpha[i] = expf(m[i] - mn);  // 0 on the first tile without a sink (m = -inf, mn finite: the tile has key lo)
+            alpha[i] = expf(m[i] - mn);  // 0 on the first tile without a sink (m = -inf, mn finite: the tile has a key)
             l[i] = l[i] * alpha[i] + wave_sum(p[i]);
             m[i] = mn;
         }
@@ -198,7 +212,7 @@ __global__ __launch_bounds__(64) void attn_rows_kernel(const void* q, int ldq, c
         for (int i = 0; i < REP; ++i) ps[i * 64 + lane] = p[i];
         rowoff[lane] = (tok * ex.gv + g % ex.gv) * dv;
         __syncthreads();
-        const int nk = min(64, pos - j0 + 1);
+        const int nk = min(64, v_end - j0);
         // VB keys' values for all of the lane's columns are requested together (clamped columns: no branch between
         // the loads), then multiplied in
         constexpr int VB = DVU <= 2 ? 16 : 4;
@@ -352,6 +366,9 @@ __global__ __launch_bounds__(256) void attn_chunk_mfma_kernel(const bf16_t* __re
     const int kv_end = p0 + min(n, q0 + RT * 16);  // one past the last visible key
     const int kt_begin = chunk > 0 ? (a_pos / chunk) * chunk : window > 0 ? max(0, a_pos - window + 1) : 0;
     const float qs = scale * LOG2E_;
+    // kept first tokens in front of the workgroup's window: tiles of their own, [0, kend1), before those from kt_begin on
+    const int kend1 = window > 0 ? min(ex.keep, kt_begin) : 0;
+    const int nt1 = (kend1 + KT - 1) / KT, ntiles = nt1 + (kv_end - kt_begin + KT - 1) / KT;
 
     bf16x8 qf[DK / 32];
     {
@@ -379,12 +396,15 @@ __global__ __launch_bounds__(256) void attn_chunk_mfma_kernel(const bf16_t* __re
 
     constexpr int KCH = KT * DK / 8 / 256, VCH = KT * DV / 8 / 256;  // 16-byte pieces per thread
     u32x4 kr[KCH], vr[VCH];
-#define LOAD_TILE(kt0_) tile_load<DK, DV, KT, 256>(kr, vr, kc, vc, table, bs, G, kvh, ex.gv, kt0_, kv_end, threadIdx.x)
+#define TILE_POS(it_) ((it_) < nt1 ? (it_) * KT : kt_begin + ((it_) - nt1) * KT)
+#define TILE_END(it_) ((it_) < nt1 ? kend1 : kv_end)
+#define LOAD_TILE(kt0_) tile_load<DK, DV, KT, 256>(kr, vr, kc, vc, table, bs, G, kvh, ex.gv, TILE_POS(kt0_), TILE_END(kt0_), threadIdx.x)
 #define STORE_TILE() tile_store<DK, DV, KT, 256, KSTR, VSTR>(kr, vr, k_lds, v_lds, threadIdx.x)
-    if (kt_begin < kv_end) LOAD_TILE(kt_begin);
-    for (int kt0 = kt_begin; kt0 < kv_end; kt0 += KT) {
+    if (ntiles > 0) LOAD_TILE(0);
+    for (int it = 0; it < ntiles; ++it) {
+        const int kt0 = TILE_POS(it), kt_end = TILE_END(it);
         STORE_TILE();
-        if (kt0 + KT < kv_end) LOAD_TILE(kt0 + KT);
+        if (it + 1 < ntiles) LOAD_TILE(it + 1);
         __syncthreads();
         // ---- S = Q K^T : 16 rows x 64 keys ----
         f32x4 sacc[4];
@@ -434,7 +454,7 @@ __global__ __launch_bounds__(256) void attn_chunk_mfma_kernel(const bf16_t* __re
             for (int t = 0; t < 4; ++t) {
                 const int kp = kt0 + 16 * t + col;
                 float v = sacc[t][i];
-                if (kp > qpos || kp < lo_row[i] || qi >= n) v = -INFINITY;
+                if (kp > qpos || (kp < lo_row[i] && kp >= ex.keep) || kp >= kt_end || qi >= n) v = -INFINITY;
                 sacc[t][i] = v;
                 mx = fmaxf(mx, v);
             }
@@ -522,11 +542,12 @@ __global__ __launch_bounds__(64) void attn_decode_mfma_kernel(const bf16_t* __re
     const int s = blockIdx.x, kvh = blockIdx.y, z = blockIdx.z;
     const int rep = H / G;
     const int qpos = ctx[s] - 1;
-    int lo = chunk > 0 ? (qpos / chunk) * chunk : window > 0 ? max(0, qpos - window + 1) : 0;
-    int kv_end = qpos + 1;
+    const int lo = chunk > 0 ? (qpos / chunk) * chunk : window > 0 ? max(0, qpos - window + 1) : 0;
+    const KeyRange kr = key_range(lo, window, ex.keep);
+    int v_begin = 0, v_end = qpos + 1 - kr.gap;  // visible keys [v_begin, v_end)
     if (parts > 1) {
-        lo += z * part_len;
-        kv_end = min(kv_end, lo + part_len);
+        v_begin = z * part_len;
+        v_end = min(v_end, v_begin + part_len);
         sink = 0;  // joins in the merge
     }
     int hrow[4];  // query head of each of the lane's result rows (rows beyond the group repeat its last head)
@@ -560,7 +581,7 @@ __global__ __launch_bounds__(64) void attn_decode_mfma_kernel(const bf16_t* __re
     auto load_tile = [&](int kt0) {
 #pragma unroll
         for (int t = 0; t < KT / 16; ++t) {
-            const int pos = min(kt0 + 16 * t + col, kv_end - 1);  // clamped: keys past the end are masked below
+            const int pos = kr.pos(min(kt0 + 16 * t + col, v_end - 1));  // clamped: keys past the end are masked below
             const bf16_t* kp = kc + (((size_t)table[pos / bs] * bs + (pos % bs)) * G + kvh) * DK + 8 * g;
 #pragma unroll
             for (int ks = 0; ks < DK / 32; ++ks) kf[t][ks] = *(const u32x4*)(kp + 32 * ks);
@@ -569,12 +590,12 @@ __global__ __launch_bounds__(64) void attn_decode_mfma_kernel(const bf16_t* __re
         for (int j = 0; j < VCH; ++j) {
             const int id = lane + j * 64;
             const int p = id / (DV / 8), c = id % (DV / 8);
-            const int pos = min(kt0 + p, kv_end - 1);
+            const int pos = kr.pos(min(kt0 + p, v_end - 1));
             vr[j] = *(const u32x4*)(vc + (((size_t)table[pos / bs] * bs + (pos % bs)) * ex.gv + kvh % ex.gv) * DV + c * 8);
         }
     };
-    if (lo < kv_end) load_tile(lo);
-    for (int kt0 = lo; kt0 < kv_end; kt0 += KT) {
+    if (v_begin < v_end) load_tile(v_begin);
+    for (int kt0 = v_begin; kt0 < v_end; kt0 += KT) {  // (kt0 counts visible keys)
         __syncthreads();  // (one wave: orders the previous tile's LDS reads before these writes)
 #pragma unroll
         for (int j = 0; j < VCH; ++j) {
@@ -590,12 +611,19 @@ __global__ __launch_bounds__(64) void attn_decode_mfma_kernel(const bf16_t* __re
                 sacc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qf[ks], __builtin_bit_cast(bf16x8, kf[t][ks]), sacc[t],
                                                                   0, 0, 0);
         }
-        if (kt0 + KT < kv_end) load_tile(kt0 + KT);
+        if (kt0 + KT < v_end) load_tile(kt0 + KT);
         // bias by distance: every row (query head) of the tile is at the same position, key 16t + col lies
-        // qpos - kt0 - col - 16t keys back; each head has its own table row
-        if (ex.bias) {
-            const int d0 = qpos - kt0 - col;
-            const bool inside = qpos - (kt0 + KT - 1) >= 0 && qpos - kt0 < ex.nb;  // wave-uniform: no clamps needed
+        // d0 - 16t keys back (a tile that begins behind the kept tokens); each head has its own table row
+        if (ex.bias && kt0 < kr.kn) {  // kept tokens and the window's first keys in one tile: distances one by one
+#pragma unroll
+            for (int t = 0; t < KT / 16; ++t) {
+                const int d = min(max(qpos - kr.pos(min(kt0 + 16 * t + col, v_end - 1)), 0), ex.nb - 1);
+#pragma unroll
+                for (int i = 0; i < 4; ++i) sacc[t][i] = sacc[t][i] * qs + ex.bias[(size_t)hrow[i] * ex.nb + d] * LOG2E_;
+            }
+        } else if (ex.bias) {
+            const int d0 = qpos - kr.gap - kt0 - col;
+            const bool inside = d0 + col - (KT - 1) >= 0 && d0 + col < ex.nb;  // wave-uniform: no clamps needed
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
                 const float* bp = ex.bias + (size_t)hrow[i] * ex.nb;
@@ -619,7 +647,7 @@ __global__ __launch_bounds__(64) void attn_decode_mfma_kernel(const bf16_t* __re
             for (int t = 0; t < KT / 16; ++t) {
                 const int kp = kt0 + 16 * t + col;
                 float v = sacc[t][i];
-                if (kp >= kv_end) v = -INFINITY;
+                if (kp >= v_end) v = -INFINITY;
                 sacc[t][i] = v;
                 mx = fmaxf(mx, v);
             }
@@ -687,6 +715,8 @@ __global__ __launch_bounds__(64) void attn_decode_mfma_kernel(const bf16_t* __re
 }
 
 #undef LOAD_TILE
+#undef TILE_POS
+#undef TILE_END
 #undef STORE_TILE
 
 // grid (rows, H): combines the partitions of a row (at most 64: lane z holds partition z's maximum and sum) in a fixed
@@ -728,13 +758,14 @@ __global__ __launch_bounds__(64) void attn_merge_kernel(const float* part_ml, co
     }
 }
 
-// grid (keys, G): key jj of the range is the token at position lo + jj of the sequence whose block table is `table`;
+// grid (keys, G): key jj of the range is the token at position lo + jj - kn of the sequence whose block table is `table`
+// (the first kn keys: positions 0 .. kn - 1, the kept first tokens in front of a window);
 // its group's key and value rows go to kh [G][n][dk] and vh [G][n][dv] (the value row of head g % Gv)
 template <typename E>
 __global__ __launch_bounds__(64) void kv_gather_kernel(const E* kc, const E* vc, int bs, const int* table, int lo, int n,
-                                                       int G, int dk, int dv, E* kh, E* vh, int Gv) {
+                                                       int G, int dk, int dv, E* kh, E* vh, int Gv, int kn) {
     const int jj = blockIdx.x, g = blockIdx.y;
-    const int j = lo + jj;
+    const int j = jj < kn ? jj : lo + jj - kn;
     const long tok = (long)table[j / bs] * bs + (j % bs);
     const E* ks = kc + (tok * G + g) * dk;
     const E* vs = vc + (tok * Gv + g % Gv) * dv;
@@ -758,24 +789,30 @@ __global__ __launch_bounds__(64) void head_transpose_kernel(const void* src, lon
 }
 
 // grid (H * n): row (h, i) holds the raw scores of the query at position p0 + i against the keys at positions
-// key0 .. key0 + nk - 1. Writes the masked, sink-normalised softmax weights (zeros outside the visible range). With
+// key0 .. key0 + nk - kn - 1, behind kn columns for the kept first tokens 0 .. kn - 1. Writes the masked, sink-normalised softmax weights (zeros outside the visible range). With
 // `two` (bf16 weights) a row of the output holds 2 nk numbers: every weight's bf16 rounding, then the bf16 roundings
 // of what the first rounding lost, so that a product with the values stacked twice sees 16 bits of each weight.
 template <bool P16>
 __global__ __launch_bounds__(256) void masked_softmax_kernel(const float* sc, void* pw, int n, int nk, int p0, int key0,
                                                              float scale, int chunk, int window, int sink,
                                                              const float* sink_v, const float* bias, int nb, int H,
-                                                             int two) {
+                                                             int two, int kn, int keep) {
     __shared__ float red[4];
     const long row = blockIdx.x;
     const int i = (int)(row % n), h = (int)(row / n);
     const int pos = p0 + i;
     const int lo = chunk > 0 ? (pos / chunk) * chunk : window > 0 ? max(0, pos - window + 1) : 0;
-    const int a = max(lo, key0) - key0, b = min(pos - key0, nk - 1);  // visible local range [a, b]
+    const int gap = key0 - kn;  // column j >= kn is the key at position j + gap
+    const bool kept = keep > 0 && window > 0;
+    // visible columns [a, b]; with kept first tokens those in front of the row's window are left out one by one
+    const int a = kept ? 0 : max(lo, key0) - gap, b = min(pos - gap, nk - 1);
     const float* s = sc + row * nk;
     const float s0 = sink_v ? sink_v[h] : 0.f;
-    const int d0 = pos - key0;  // distance of local key j: d0 - j
-    auto score = [&](int j) { return s[j] * scale + (bias ? bias[(long)h * nb + min(d0 - j, nb - 1)] : 0.f); };
+    auto score = [&](int j) {
+        const int p = j < kn ? j : j + gap;
+        if (p < lo && p >= keep) return -INFINITY;
+        return s[j] * scale + (bias ? bias[(long)h * nb + min(pos - p, nb - 1)] : 0.f);
+    };
     float m = sink ? s0 : -INFINITY;
     for (int j = a + threadIdx.x; j <= b; j += 256) m = fmaxf(m, score(j));
     m = block_max<256>(m, red);
@@ -809,10 +846,10 @@ extern "C" int mxh_attention(const void* q, int ldq, int q16, const void* kc, co
                              void* out, int ldo, int o16, int H, int G, int dk, int dv, float scale, int chunk,
                              int window, int sink, float out_scale, int row_off, int parts, int part_len,
                              float* part_ml, float* part_o, const float* sink_v, const float* bias, int nb,
-                             const float* gate, int ldg, int gv, hipStream_t st) {
+                             const float* gate, int ldg, int gv, int keep, hipStream_t st) {
     if (n_rows <= 0 || n_seqs <= 0) return 0;
-    MXH_CHECK((!bias || nb > 0) && (!gate || ldg >= H) && (!sink_v || sink) && gv > 0 && G % gv == 0);
-    const AttnExtra ex = {sink_v, bias, nb, gate, ldg, gv};
+    MXH_CHECK((!bias || nb > 0) && (!gate || ldg >= H) && (!sink_v || sink) && gv > 0 && G % gv == 0 && keep >= 0);
+    const AttnExtra ex = {sink_v, bias, nb, gate, ldg, gv, keep};
     MXH_CHECK(q && kc && vc && bt && ctx && out && bs > 0 && bt_stride > 0);
     MXH_CHECK(H > 0 && G > 0 && H % G == 0 && dk > 0 && dv > 0 && dv <= 64 * DVU_MAX && dk <= 4096);
     MXH_CHECK(ldq >= H * dk && ldo >= H * dv && chunk >= 0 && window >= 0 && H <= 65535 && row_off >= 0);
@@ -848,15 +885,15 @@ extern "C" int mxh_attention(const void* q, int ldq, int q16, const void* kc, co
 }
 
 extern "C" int mxh_kv_gather(const void* kc, const void* vc, int is16, int bs, const int* table, int lo, int n, int G,
-                             int dk, int dv, void* kh, void* vh, int Gv, hipStream_t st) {
+                             int dk, int dv, void* kh, void* vh, int Gv, int kn, hipStream_t st) {
     if (n <= 0) return 0;
     MXH_CHECK(kc && vc && table && kh && vh && bs > 0 && lo >= 0 && G > 0 && G <= 65535 && dk > 0 && dv > 0);
-    MXH_CHECK(Gv > 0 && G % Gv == 0);
+    MXH_CHECK(Gv > 0 && G % Gv == 0 && kn >= 0 && kn <= lo && kn <= n);
     const dim3 grid(n, G);
     if (is16) kv_gather_kernel<bf16_t><<<grid, 64, 0, st>>>((const bf16_t*)kc, (const bf16_t*)vc, bs, table, lo, n, G, dk,
-                                                           dv, (bf16_t*)kh, (bf16_t*)vh, Gv);
+                                                           dv, (bf16_t*)kh, (bf16_t*)vh, Gv, kn);
     else kv_gather_kernel<float><<<grid, 64, 0, st>>>((const float*)kc, (const float*)vc, bs, table, lo, n, G, dk, dv,
-                                                      (float*)kh, (float*)vh, Gv);
+                                                      (float*)kh, (float*)vh, Gv, kn);
     return (int)hipGetLastError();
 }
 
@@ -877,17 +914,17 @@ extern "C" int mxh_head_transpose(const void* src, int s16, long s_si, long s_sh
 
 extern "C" int mxh_masked_softmax(const float* sc, void* pw, int p16, long rows, int n, int nk, int p0, int key0,
                                   float scale, int chunk, int window, int sink, const float* sink_v,
-                                  const float* bias, int nb, int H, int two, hipStream_t st) {
+                                  const float* bias, int nb, int H, int two, int kn, int keep, hipStream_t st) {
     if (rows <= 0) return 0;
-    MXH_CHECK(!two || p16);
+    MXH_CHECK((!two || p16) && kn >= 0 && kn <= key0 && kn <= nk && keep >= 0);
     MXH_CHECK(sc && pw && n > 0 && nk > 0 && rows % n == 0 && rows < (1L << 31) && key0 >= 0 && p0 >= key0);
     MXH_CHECK((!bias || nb > 0) && (!(bias || sink_v) || rows == (long)H * n));
     if (p16)
         masked_softmax_kernel<true><<<(unsigned)rows, 256, 0, st>>>(sc, pw, n, nk, p0, key0, scale, chunk, window, sink,
-                                                                    sink_v, bias, nb, H, two);
+                                                                    sink_v, bias, nb, H, two, kn, keep);
     else
         masked_softmax_kernel<false><<<(unsigned)rows, 256, 0, st>>>(sc, pw, n, nk, p0, key0, scale, chunk, window, sink,
-                                                                     sink_v, bias, nb, H, 0);
+                                                                     sink_v, bias, nb, H, 0, kn, keep);
     return (int)hipGetLastError();
 }
 
@@ -899,10 +936,10 @@ extern "C" int mxh_attention_mfma(const void* q, int ldq, const void* kc, const 
                                   int p0, int n, void* out, int ldo, int o16, int H, int G, int dk, int dv,
                                   float scale, int chunk, int window, int sink, float out_scale, const float* sink_v,
                                   const float* bias, int nb, const float* gate, int ldg, int gv, int p2,
-                                  hipStream_t st) {
+                                  int keep, hipStream_t st) {
     if (n <= 0) return 0;
-    MXH_CHECK((!bias || nb > 0) && (!gate || ldg >= H) && (!sink_v || sink) && gv > 0 && G % gv == 0);
-    const AttnExtra ex = {sink_v, bias, nb, gate, ldg, gv};
+    MXH_CHECK((!bias || nb > 0) && (!gate || ldg >= H) && (!sink_v || sink) && gv > 0 && G % gv == 0 && keep >= 0);
+    const AttnExtra ex = {sink_v, bias, nb, gate, ldg, gv, keep};
     MXH_CHECK(q && kc && vc && table && out && bs > 0 && p0 >= 0 && H > 0 && G > 0 && H % G == 0);
     MXH_CHECK(mxh_attention_mfma_ok(dk, dv) && ldq >= H * dk && ldq % 8 == 0 && ldo >= H * dv && chunk >= 0 && window >= 0);
     const int rep = H / G;
@@ -937,10 +974,10 @@ extern "C" int mxh_attention_decode_mfma(const void* q, int ldq, const void* kc,
                                          int G, int dk, int dv, float scale, int chunk, int window, int sink,
                                          float out_scale, int parts, int part_len, float* part_ml, float* part_o,
                                          const float* sink_v, const float* bias, int nb, const float* gate, int ldg,
-                                         int gv, int p2, hipStream_t st) {
+                                         int gv, int p2, int keep, hipStream_t st) {
     if (n_seqs <= 0) return 0;
-    MXH_CHECK((!bias || nb > 0) && (!gate || ldg >= H) && (!sink_v || sink) && gv > 0 && G % gv == 0);
-    const AttnExtra ex = {sink_v, bias, nb, gate, ldg, gv};
+    MXH_CHECK((!bias || nb > 0) && (!gate || ldg >= H) && (!sink_v || sink) && gv > 0 && G % gv == 0 && keep >= 0);
+    const AttnExtra ex = {sink_v, bias, nb, gate, ldg, gv, keep};
     MXH_CHECK(q && kc && vc && bt && ctx && out && bs > 0 && bt_stride > 0 && H > 0 && G > 0 && H % G == 0);
     MXH_CHECK(H / G <= 16 && G <= 65535 && mxh_attention_mfma_ok(dk, dv) && ldq >= H * dk && ldq % 8 == 0 && ldo >= H * dv);
     MXH_CHECK(parts >= 1 && parts <= 64 && (parts == 1 || (part_len > 0 && part_ml && part_o)) && chunk >= 0 && window >= 0);

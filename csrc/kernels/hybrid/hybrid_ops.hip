@@ -1,5 +1,6 @@
 // hybrid_ops.hip: the fp32 row kernels of hybrid attention / recurrent decoders (ops/hybrid.py): embedding gather,
-// offset RMS norm, output norm + residual add, rotary + head norm (+ weights, query temperature) + paged append, causal
+// offset RMS norm, output norm + residual add, scaled residual add + the norm that follows, rotary (+ projection biases,
+// given frequencies) + head norm (+ weights, query temperature) + paged append, causal
 // convolution with carried tails, unit-length heads, decay / write-strength coefficients, per-channel decays, gated
 // group norm, gated linear unit with per-group factors, expert routing.
 //
@@ -41,14 +42,15 @@ MX_DEV float block_sum_dyn(float v, float* red) {
 
 template <bool B16>
 __global__ __launch_bounds__(NT) void embed_rows_kernel(const void* table, int V, const int* tokens, float* out,
-                                                        int ldo, int accumulate, int C, bf16_t* o16, int ld16) {
+                                                        int ldo, int accumulate, int C, bf16_t* o16, int ld16,
+                                                        float scale) {
     const int t = blockIdx.x;
     int tok = tokens[t];
     if (tok < 0 || tok >= V) tok = 0;
     const long base = (long)tok * C;
     float* o = out + (long)t * ldo;
     for (int c = threadIdx.x; c < C; c += NT) {
-        float v = ld_elem<B16>(table, base + c);
+        float v = ld_elem<B16>(table, base + c) * scale;
         if (accumulate) v += o[c];
         o[c] = v;
         if (o16) o16[(long)t * ld16 + c] = f32_to_bf16(v);
@@ -151,9 +153,73 @@ __global__ __launch_bounds__(1024) void norm_add_kernel(const float* y, int ldy,
     }
 }
 
+// x[t] += (y[t] + b) * s (b, s per column, either may be null: 0 / 1); with w also the norm that follows,
+// h = x[t] / rms(x[t]) * (offset + w), as fp32 and / or bf16. One block per row (256 or 1024 threads); rows of up to
+// nt * RK numbers keep the new x in registers between the two.
+template <int RK>
+__global__ __launch_bounds__(1024) void scale_add_norm_kernel(const float* y, int ldy, const float* b, const float* s,
+                                                              float* x, int ldx, const float* w, float offset, float eps,
+                                                              float* o32, int ld32, bf16_t* o16, int ld16, int C) {
+    __shared__ float red[16];
+    const int i = blockIdx.x, nt = blockDim.x;
+    const float* yr = y + (long)i * ldy;
+    float* xr = x + (long)i * ldx;
+    const bool cached = C <= nt * RK;
+    float xk[RK], wk[RK];
+    float ss = 0.f;
+    if (cached) {
+        float yk[RK], bk[RK], sk[RK];
+#pragma unroll
+        for (int k = 0; k < RK; ++k) {  // clamped addresses: straight-line loads, all in flight together
+            const int c = min((int)threadIdx.x + k * nt, C - 1);
+            yk[k] = yr[c];
+            xk[k] = xr[c];
+            bk[k] = b ? b[c] : 0.f;
+            sk[k] = s ? s[c] : 1.f;
+            wk[k] = w ? w[c] : 0.f;
+        }
+#pragma unroll
+        for (int k = 0; k < RK; ++k) {
+            const int c = threadIdx.x + k * nt;
+            xk[k] += (yk[k] + bk[k]) * sk[k];
+            if (c < C) {
+                xr[c] = xk[k];
+                ss += xk[k] * xk[k];
+            }
+        }
+    } else {
+        for (int c = threadIdx.x; c < C; c += nt) {
+            const float v = xr[c] + (yr[c] + (b ? b[c] : 0.f)) * (s ? s[c] : 1.f);
+            xr[c] = v;
+            ss += v * v;
+        }
+    }
+    if (!w) return;
+    ss = block_sum_dyn(ss, red);
+    const float sc = 1.f / sqrtf(ss / (float)C + eps);
+    if (cached) {
+#pragma unroll
+        for (int k = 0; k < RK; ++k) {
+            const int c = threadIdx.x + k * nt;
+            if (c < C) {
+                const float v = xk[k] * sc * (offset + wk[k]);
+                if (o32) o32[(long)i * ld32 + c] = v;
+                if (o16) o16[(long)i * ld16 + c] = f32_to_bf16(v);
+            }
+        }
+        return;
+    }
+    for (int c = threadIdx.x; c < C; c += nt) {  // (a thread reads back the columns it wrote itself)
+        const float v = xr[c] * sc * (offset + w[c]);
+        if (o32) o32[(long)i * ld32 + c] = v;
+        if (o16) o16[(long)i * ld16 + c] = f32_to_bf16(v);
+    }
+}
+
 // grid (T, H + G + Gv), one wave per (token, head): query heads, then key heads, then the Gv value heads. Element
 // e < rot_dims of a query / key head turns with its neighbour e ^ 1 by angle pos * base^(-(e / 2) * 2 / rot_dims); with
-// `half` the pairs are (i, i + rot_dims / 2) instead and pair i turns by pos * base^(-i * 2 / rot_dims).
+// `half` the pairs are (i, i + rot_dims / 2) instead and pair i turns by pos * base^(-i * 2 / rot_dims). Given `freqs`
+// (one per pair) pair i turns by pos * freqs[i]; sine and cosine are multiplied by mag. qb, kb, vb: projection biases.
 constexpr int HEAD_E = 8;  // elements per lane: heads of up to 512 numbers
 template <bool Q16, bool C16>
 __global__ __launch_bounds__(64) void rope_norm_append_kernel(const float* qi, const float* ki, const float* vi,
@@ -162,7 +228,8 @@ __global__ __launch_bounds__(64) void rope_norm_append_kernel(const float* qi, c
                                                               int norm, float eps, void* qo, int ldqo, void* kc,
                                                               void* vc, const int* slots, const float* qw,
                                                               const float* kw, float temp_coef, int temp_every,
-                                                              int half, int Gv) {
+                                                              int half, int Gv, const float* freqs, float mag,
+                                                              const float* qb, const float* kb, const float* vb) {
     const int t = blockIdx.x, u = blockIdx.y, lane = threadIdx.x;
     if (u >= H + G) {  // value head: plain copy into the pool
         const int sl = slots[t];
@@ -170,7 +237,7 @@ __global__ __launch_bounds__(64) void rope_norm_append_kernel(const float* qi, c
         const int g = u - H - G;
         const float* src = vi + (long)t * ldv + (long)g * dv;
         const long dst = ((long)sl * Gv + g) * dv;
-        for (int e = lane; e < dv; e += 64) st_elem<C16>(vc, dst + e, src[e]);
+        for (int e = lane; e < dv; e += 64) st_elem<C16>(vc, dst + e, src[e] + (vb ? vb[g * dv + e] : 0.f));
         return;
     }
     const bool isq = u < H;
@@ -181,6 +248,8 @@ __global__ __launch_bounds__(64) void rope_norm_append_kernel(const float* qi, c
         if (sl < 0) return;
     }
     const float* src = isq ? qi + (long)t * ldq + (long)hd * dk : ki + (long)t * ldk + (long)hd * dk;
+    const float* hb = isq ? qb : kb;
+    if (hb) hb += (long)hd * dk;
     const float pos = (float)positions[t];
     float val[HEAD_E];
     float ss = 0.f;
@@ -189,16 +258,18 @@ __global__ __launch_bounds__(64) void rope_norm_append_kernel(const float* qi, c
         const int e = lane + k * 64;
         float v = 0.f;
         if (e < dk) {
-            v = src[e];
+            v = src[e] + (hb ? hb[e] : 0.f);
             if (e < rot) {
                 const int n2 = rot >> 1;
                 const bool second = half ? e >= n2 : (e & 1);  // the pair's second member turns as v cos + u sin
                 const int mate = half ? (second ? e - n2 : e + n2) : (e ^ 1);
                 const int pi = half ? (second ? e - n2 : e) : (e >> 1);
-                const float other = src[mate];
-                const float f = expf((float)pi * (2.f / (float)rot) * neg_log_base);
+                const float other = src[mate] + (hb ? hb[mate] : 0.f);
+                const float f = freqs ? freqs[pi] : expf((float)pi * (2.f / (float)rot) * neg_log_base);
                 float s, c;
                 sincosf(pos * f, &s, &c);
+                s *= mag;
+                c *= mag;
                 v = second ? v * c + other * s : v * c - other * s;
             }
         }
@@ -429,14 +500,16 @@ __global__ void gated_group_norm_kernel(const float* y, int ldy, const float* ga
 }
 
 // grid (T, ceil(F / NT))
-// act 0: silu(x) * y * factor; 1: gelu_tanh(x) * y * factor; 2 (no second operand): relu(factor * x)^2
+// act 0: silu(x) * y * factor; 1: gelu_tanh(x) * y * factor; 2 (no second operand): relu(factor * x)^2;
+// 3: g sigmoid(alpha g) (u + 1) * factor with g = min(x, limit), u = clamp(y, -limit, limit)
 MX_DEV float gelu_tanh_acc(float x) {
     return 0.5f * x * (1.f + tanhf(0.7978845608028654f * (x + 0.044715f * x * x * x)));
 }
 template <bool B16>
 __global__ __launch_bounds__(NT) void glu_kernel(const float* a, int lda, const float* b, int ldb, const float* ba,
                                                  const float* bb, const float* scale, int lds, int group,
-                                                 int scale_sigmoid, void* out, int ldo, int F, int act) {
+                                                 int scale_sigmoid, void* out, int ldo, int F, int act, float limit,
+                                                 float alpha) {
     const int f = blockIdx.y * NT + threadIdx.x, t = blockIdx.x;
     if (f >= F) return;
     float fac = 1.f;
@@ -455,14 +528,23 @@ __global__ __launch_bounds__(NT) void glu_kernel(const float* a, int lda, const 
         return;
     }
     const float y = b[(long)t * ldb + f] + (bb ? bb[f] : 0.f);
+    if (act == 3) {
+        const float g = fminf(x, limit), u = fminf(fmaxf(y, -limit), limit);
+        st_elem<B16>(out, (long)t * ldo + f, g * sigmoid_acc(alpha * g) * (u + 1.f) * fac);
+        return;
+    }
     st_elem<B16>(out, (long)t * ldo + f, (act == 1 ? gelu_tanh_acc(x) : silu_acc(x)) * y * fac);
 }
 
 // one wave per token; lane l holds experts l, l + 64, ... (up to 16 each)
 constexpr int ROUTE_E = 16;
-// sigm: the chosen experts keep sigmoid(logit) * scale as their weights (no softmax, no renormalisation)
+// mode 0: the chosen experts' softmax scores are renormalised; 1: they keep sigmoid(logit) * scale; 2: they keep their
+// softmax score over all experts, times scale. With `groups` > 1 the experts form that many equal groups of neighbours
+// and only the experts of the `gkeep` groups with the largest best scores can be chosen (ties: the lower group).
 __global__ __launch_bounds__(64) void moe_route_kernel(const float* logits, int ld, const float* bias, int E, int top,
-                                                       float scale, float eps, float* weights, int sigm) {
+                                                       float scale, float eps, float* weights, int mode, int groups,
+                                                       int gkeep) {
+    extern __shared__ float sh[];  // [E] scores, [groups] best scores (with groups only)
     const int t = blockIdx.x, lane = threadIdx.x;
     const float* z = logits + (long)t * ld;
     float v[ROUTE_E];
@@ -483,6 +565,31 @@ __global__ __launch_bounds__(64) void moe_route_kernel(const float* logits, int 
     sum = wave_sum(sum);
     float* wr = weights + (long)t * E;
     for (int e = lane; e < E; e += 64) wr[e] = 0.f;
+    unsigned taken = 0;  // bit k: expert lane + 64 k was chosen
+    if (groups > 1) {
+        float* gm = sh + E;
+        const int per = E / groups;
+#pragma unroll
+        for (int k = 0; k < ROUTE_E; ++k)
+            if (lane + k * 64 < E) sh[lane + k * 64] = v[k];
+        __syncthreads();
+        for (int g = lane; g < groups; g += 64) {
+            float best = sh[g * per];
+            for (int i = 1; i < per; ++i) best = fmaxf(best, sh[g * per + i]);
+            gm[g] = best;
+        }
+        __syncthreads();
+#pragma unroll
+        for (int k = 0; k < ROUTE_E; ++k) {
+            const int e = lane + k * 64;
+            if (e < E) {
+                const int g = e / per;
+                int better = 0;  // groups ahead of this expert's
+                for (int o = 0; o < groups; ++o) better += gm[o] > gm[g] || (gm[o] == gm[g] && o < g);
+                if (better >= gkeep) v[k] = -1.f;
+            }
+        }
+    }
     float mine[ROUTE_E];  // score of the experts this lane holds that were chosen (else 0)
 #pragma unroll
     for (int k = 0; k < ROUTE_E; ++k) mine[k] = 0.f;
@@ -512,6 +619,7 @@ __global__ __launch_bounds__(64) void moe_route_kernel(const float* logits, int 
             if (lane + k * 64 == bi) {
                 mine[k] = v[k] / sum;
                 v[k] = -1.f;
+                taken |= 1u << k;
             }
         }
     }
@@ -519,9 +627,9 @@ __global__ __launch_bounds__(64) void moe_route_kernel(const float* logits, int 
 #pragma unroll
     for (int k = 0; k < ROUTE_E; ++k) {
         const int e = lane + k * 64;
-        if (e < E && v[k] < 0.f) {  // the taken ones (absent ones have e >= E)
-            // exp(z - m) orders the experts as their logits do, so the same `top` are taken in both modes
-            wr[e] = sigm ? scale * sigmoid_acc(z[e] + (bias ? bias[e] : 0.f)) : mine[k] * norm;
+        if (taken >> k & 1u) {
+            // exp(z - m) orders the experts as their logits do, so the same `top` are taken in every mode
+            wr[e] = mode == 1 ? scale * sigmoid_acc(z[e] + (bias ? bias[e] : 0.f)) : mine[k] * (mode == 2 ? scale : norm);
         }
     }
 }
@@ -532,11 +640,11 @@ __global__ __launch_bounds__(64) void moe_route_kernel(const float* logits, int 
     if (!(cond)) return (int)hipErrorInvalidValue
 
 extern "C" int mxh_embed_rows(const void* table, int is16, int V, const int* tokens, float* out, int ldo,
-                              int accumulate, bf16_t* o16, int ld16, int T, int C, hipStream_t st) {
+                              int accumulate, bf16_t* o16, int ld16, float scale, int T, int C, hipStream_t st) {
     if (T <= 0) return 0;
     MXH_CHECK(table && tokens && out && C > 0 && V > 0 && ldo >= C && (!o16 || ld16 >= C));
-    if (is16) embed_rows_kernel<true><<<T, NT, 0, st>>>(table, V, tokens, out, ldo, accumulate, C, o16, ld16);
-    else embed_rows_kernel<false><<<T, NT, 0, st>>>(table, V, tokens, out, ldo, accumulate, C, o16, ld16);
+    if (is16) embed_rows_kernel<true><<<T, NT, 0, st>>>(table, V, tokens, out, ldo, accumulate, C, o16, ld16, scale);
+    else embed_rows_kernel<false><<<T, NT, 0, st>>>(table, V, tokens, out, ldo, accumulate, C, o16, ld16, scale);
     return (int)hipGetLastError();
 }
 
@@ -558,11 +666,25 @@ extern "C" int mxh_norm_add(const float* y, int ldy, const float* w, float offse
     return (int)hipGetLastError();
 }
 
+extern "C" int mxh_scale_add_norm(const float* y, int ldy, const float* b, const float* s, float* x, int ldx,
+                                  const float* w, float offset, float eps, float* o32, int ld32, bf16_t* o16, int ld16,
+                                  int T, int C, hipStream_t st) {
+    if (T <= 0) return 0;
+    MXH_CHECK(y && x && C > 0 && ldy >= C && ldx >= C && (!w || o32 || o16) && (!o32 || ld32 >= C) && (!o16 || ld16 >= C));
+#define GO(K_, nt_) scale_add_norm_kernel<K_><<<T, nt_, 0, st>>>(y, ldy, b, s, x, ldx, w, offset, eps, o32, ld32, o16, ld16, C)
+    if (C <= 1024) GO(4, 256);
+    else if (C <= 4096) GO(4, 1024);
+    else GO(8, 1024);
+#undef GO
+    return (int)hipGetLastError();
+}
+
 extern "C" int mxh_rope_norm_append(const float* qi, const float* ki, const float* vi, int ldq, int ldk, int ldv,
                                     const int* positions, int H, int G, int dk, int dv, int rot, float base, int norm,
                                     float eps, void* qo, int ldqo, int q16, void* kc, void* vc, int c16,
                                     const int* slots, const float* qw, const float* kw, float temp_coef,
-                                    int temp_every, int half, int Gv, int T, hipStream_t st) {
+                                    int temp_every, int half, int Gv, const float* freqs, float mag, const float* qb,
+                                    const float* kb, const float* vb, int T, hipStream_t st) {
     if (T <= 0) return 0;
     MXH_CHECK(qi && ki && vi && positions && qo && kc && vc && slots && temp_every >= 1);
     // G == 0: queries only (keys and values of another layer are read). Gv value heads (the pool's row is Gv * dv)
@@ -574,7 +696,7 @@ extern "C" int mxh_rope_norm_append(const float* qi, const float* ki, const floa
 #define GO(Q, C)                                                                                                   \
     rope_norm_append_kernel<Q, C><<<grid, 64, 0, st>>>(qi, ki, vi, ldq, ldk, ldv, positions, H, G, dk, dv, rot, nlb, \
                                                        norm, eps, qo, ldqo, kc, vc, slots, qw, kw, temp_coef, temp_every, \
-                                                       half, Gv)
+                                                       half, Gv, freqs, mag, qb, kb, vb)
     if (q16 && c16) GO(true, true);
     else if (q16) GO(true, false);
     else if (c16) GO(false, true);
@@ -653,23 +775,28 @@ extern "C" int mxh_gated_group_norm(const float* y, int ldy, const float* gate, 
 
 extern "C" int mxh_glu(const float* a, int lda, const float* b, int ldb, const float* ba, const float* bb,
                        const float* scale, int lds, int group, int scale_sigmoid, void* out, int ldo, int o16, int T,
-                       int F, int act, hipStream_t st) {
+                       int F, int act, float limit, float alpha, hipStream_t st) {
     if (T <= 0 || F <= 0) return 0;
-    MXH_CHECK(a && out && lda >= F && ldo >= F && group > 0 && F <= 65535 * NT && act >= 0 && act <= 2);
+    MXH_CHECK(a && out && lda >= F && ldo >= F && group > 0 && F <= 65535 * NT && act >= 0 && act <= 3);
     MXH_CHECK(act == 2 ? !b : (b && ldb >= F));  // the squared ReLU has one operand
     MXH_CHECK(!scale || (F % group == 0 && lds >= F / group));
     const dim3 grid(T, (F + NT - 1) / NT);
     if (o16)
-        glu_kernel<true><<<grid, NT, 0, st>>>(a, lda, b, ldb, ba, bb, scale, lds, group, scale_sigmoid, out, ldo, F, act);
+        glu_kernel<true><<<grid, NT, 0, st>>>(a, lda, b, ldb, ba, bb, scale, lds, group, scale_sigmoid, out, ldo, F, act,
+                                          limit, alpha);
     else
-        glu_kernel<false><<<grid, NT, 0, st>>>(a, lda, b, ldb, ba, bb, scale, lds, group, scale_sigmoid, out, ldo, F, act);
+        glu_kernel<false><<<grid, NT, 0, st>>>(a, lda, b, ldb, ba, bb, scale, lds, group, scale_sigmoid, out, ldo, F, act,
+                                          limit, alpha);
     return (int)hipGetLastError();
 }
 
 extern "C" int mxh_moe_route(const float* logits, int ld, const float* bias, int T, int E, int top, float scale,
-                             float eps, float* weights, int sigm, hipStream_t st) {
+                             float eps, float* weights, int mode, int groups, int gkeep, hipStream_t st) {
     if (T <= 0) return 0;
     MXH_CHECK(logits && weights && E > 0 && E <= 64 * ROUTE_E && top > 0 && top <= E && ld >= E);
-    moe_route_kernel<<<T, 64, 0, st>>>(logits, ld, bias, E, top, scale, eps, weights, sigm);
+    MXH_CHECK(mode >= 0 && mode <= 2 && groups >= 1 && E % groups == 0 && gkeep >= 1 && gkeep <= groups &&
+              top <= gkeep * (E / groups));
+    moe_route_kernel<<<T, 64, groups > 1 ? (E + groups) * sizeof(float) : 0, st>>>(logits, ld, bias, E, top, scale, eps,
+                                                                                  weights, mode, groups, gkeep);
     return (int)hipGetLastError();
 }

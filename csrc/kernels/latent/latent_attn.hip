@@ -1,6 +1,9 @@
 // latent_attn.hip: causal softmax attention over a paged pool of per-token latents, in the weight-absorbed form:
 // the rows are absorbed queries qa (one per token and head, `R` numbers), and a cached latent c_j serves as key AND
 // value for every head:   out[row] = sum_j softmax_j(qa[row] . c_j) c_j   over the keys j <= the row's position.
+// A cached row may be wider than the latent (`W` >= `R` numbers: the latent followed by a part that only keys have, for
+// instance rotated numbers shared by the heads): scores run over all W numbers, values are the first R. An optional
+// learned `sink` per head is one more score in the softmax denominator, without a value.
 //
 // One kernel serves decode rows (one token per sequence, optionally split over key partitions that a second kernel
 // merges) and prompt chunks (several tokens per sequence, causal inside the chunk). A workgroup owns BM consecutive
@@ -30,7 +33,7 @@ struct AttnArgs {
     const void* qa;
     long qs_t, qs_h;
     const void* cache;
-    int bs, R;
+    int bs, W, R;  // numbers per cached row (keys), of which the first R are the value
     const int* bt;
     int bt_stride;
     const int* cu_q;  // null: one row per sequence (decode)
@@ -42,6 +45,7 @@ struct AttnArgs {
     int H, parts, part_len;
     float* part_ml;
     float* part_o;
+    const float* sink;  // [H] or null
 };
 
 template <bool B16, int RV, int BN, int BM>
@@ -52,7 +56,7 @@ __global__ __launch_bounds__(BM * 8) void latent_attn_kernel(AttnArgs a) {
     float* CT = QA + BM * RP;        // [BN][RP]
     float* PS = CT + BN * RP;        // [BM][BN + 1]
     const int tid = threadIdx.x, m = tid >> 3, l8 = tid & 7;
-    const int H = a.H, R = a.R;
+    const int H = a.H, R = a.R, W = a.W;
 
     // ---- which sequence and which of its (token, head) rows ----
     int seq = -1, g0 = 0, qlen = 1, crow0 = 0;
@@ -99,14 +103,16 @@ __global__ __launch_bounds__(BM * 8) void latent_attn_kernel(AttnArgs a) {
         const int mm = i / RW, r = i - mm * RW;
         const int gg = g0 + mm;
         float v = 0.f;
-        if (gg < qlen * H && r < R) {
+        if (gg < qlen * H && r < W) {
             const int t2 = gg / H, h2 = gg - t2 * H;
             v = ldf<B16>(a.qa, ((long)a.row_base + crow0 + t2) * a.qs_t + (long)h2 * a.qs_h + r) * a.scale;
         }
         QA[mm * RP + r] = v;
     }
 
-    float m_run = -INFINITY, l_run = 0.f;
+    // the sink: a running maximum and sum that start at its score and 1 (partitions: it joins in the merge)
+    const bool snk = a.sink && valid && a.parts == 1;
+    float m_run = snk ? a.sink[hh] : -INFINITY, l_run = snk ? 1.f : 0.f;
     f32x4 acc[RV];
 #pragma unroll
     for (int i = 0; i < RV; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
@@ -118,9 +124,9 @@ __global__ __launch_bounds__(BM * 8) void latent_attn_kernel(AttnArgs a) {
             const int j = i / RW, r = i - j * RW;
             const int key = k0 + j;
             float v = 0.f;
-            if (key < k_end && r < R) {
+            if (key < k_end && r < W) {
                 const int blk = btr[key / a.bs];
-                v = ldf<B16>(a.cache, ((long)blk * a.bs + (key % a.bs)) * R + r);
+                v = ldf<B16>(a.cache, ((long)blk * a.bs + (key % a.bs)) * W + r);
             }
             CT[j * RP + r] = v;
         }
@@ -212,7 +218,7 @@ __global__ __launch_bounds__(BM * 8) void latent_attn_kernel(AttnArgs a) {
 template <bool B16>
 __global__ __launch_bounds__(256) void latent_attn_merge_kernel(const float* part_ml, const float* part_o, int parts,
                                                                 int R, int H, int row_base, void* out, long os_t,
-                                                                long os_h) {
+                                                                long os_h, const float* sink) {
     __shared__ float wgt[1024];
     __shared__ float red[8];
     const int seq = blockIdx.x / H, hh = blockIdx.x - seq * H;
@@ -228,7 +234,9 @@ __global__ __launch_bounds__(256) void latent_attn_merge_kernel(const float* par
     for (int o = 32; o > 0; o >>= 1) mloc = fmaxf(mloc, __shfl_xor(mloc, o, 64));
     if (lane == 0) red[wv] = mloc;
     __syncthreads();
-    const float M = fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3]));
+    float M = fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3]));
+    const float s0 = sink ? sink[hh] : -INFINITY;
+    M = fmaxf(M, s0);
     float lloc = 0.f;
     for (int p = tid; p < parts; p += 256) {
         const float mp = wgt[p];
@@ -240,7 +248,7 @@ __global__ __launch_bounds__(256) void latent_attn_merge_kernel(const float* par
     for (int o = 32; o > 0; o >>= 1) lloc += __shfl_xor(lloc, o, 64);
     if (lane == 0) red[4 + wv] = lloc;
     __syncthreads();
-    const float L = red[4] + red[5] + red[6] + red[7];
+    const float L = red[4] + red[5] + red[6] + red[7] + (sink ? __expf(s0 - M) : 0.f);
     const float inv = L > 0.f ? 1.f / L : 0.f;
     for (int c = tid; c < R; c += 256) {
         float o = 0.f;
@@ -263,7 +271,7 @@ int launch(const AttnArgs& a, int n_rows, hipStream_t st) {
 
 template <bool B16>
 int dispatch(const AttnArgs& a, int n_rows, hipStream_t st) {
-    const int rv = (a.R + 31) / 32;
+    const int rv = (a.W + 31) / 32;
     if (rv <= 1) return launch<B16, 1, 64, 32>(a, n_rows, st);
     if (rv <= 2) return launch<B16, 2, 64, 32>(a, n_rows, st);
     if (rv <= 3) return launch<B16, 3, 64, 32>(a, n_rows, st);
@@ -272,10 +280,11 @@ int dispatch(const AttnArgs& a, int n_rows, hipStream_t st) {
     if (rv <= 8) return launch<B16, 8, 16, 32>(a, n_rows, st);
     if (rv <= 12) return launch<B16, 12, 8, 16>(a, n_rows, st);
     if (rv <= 16) return launch<B16, 16, 8, 16>(a, n_rows, st);
+    if (rv <= 20) return launch<B16, 20, 8, 16>(a, n_rows, st);
     return (int)hipErrorInvalidValue;
 }
 
-// ---- the same attention on the matrix cores (bf16 storage, R a multiple of 8) ----------------------------------
+// ---- the same attention on the matrix cores (bf16 storage, W a multiple of 8) ----------------------------------
 // A workgroup of NW waves owns 16 NW consecutive (token, head) rows of one sequence; wave w holds rows 16 w .. + 15
 // as MFMA 16x16x32 A fragments (absorbed queries, read once from HBM into registers). The visible keys stream in
 // tiles of 32 latents through ONE LDS image [32][R_pad] shared by the waves, and the image serves both products:
@@ -299,18 +308,19 @@ MX_DEV float group_sum16(float v) {
 // RS = 2 splits the rank between two waves of a row tile: both compute the tile's full scores and softmax (no
 // exchange, no extra barrier), each accumulates and writes one half of the output columns. Half the accumulators per
 // wave let two waves share a SIMD at the widest ranks, which is what hides the latencies between a tile's steps.
-template <int RV, int NW, int RS>
+// NVT: 16-column tiles of the value part (NVT * 16 >= R; all of the row unless the row has many key-only numbers).
+template <int RV, int NVT, int NW, int RS>
 __global__ __launch_bounds__(NW * 64) __attribute__((amdgpu_waves_per_eu(RS == 2 ? 2 : 1)))
 void latent_attn_mfma_kernel(AttnArgs a) {
     constexpr int RP = RV * 32, KT = 32, CSTR = RP * 2 + 16, PSTR = KT * 2 + 16, NTH = NW * 64;
-    constexpr int BM = NW / RS * 16, NO = RV * 2 / RS;  // rows per workgroup, output column tiles per wave
-    static_assert(NW % RS == 0 && (RV * 2) % RS == 0, "rank split");
+    constexpr int BM = NW / RS * 16, NO = NVT / RS;  // rows per workgroup, output column tiles per wave
+    static_assert(NW % RS == 0 && NVT % RS == 0 && NVT <= RV * 2, "rank split");
     extern __shared__ __attribute__((aligned(16))) char smem[];
     char* c_lds = smem;                                   // [KT][CSTR] bf16 latents of the tile
     const int tid = threadIdx.x, wv = tid >> 6, lane = tid & 63, col = lane & 15, g = lane >> 4;
     const int wave = wv / RS, half = wv % RS;  // row tile of this wave, and which part of the rank it accumulates
     char* pw = smem + KT * CSTR + wv * 16 * PSTR;       // this wave's P [16][PSTR]
-    const int H = a.H, R = a.R;
+    const int H = a.H, R = a.R, W = a.W;
     const bf16_t* qa = (const bf16_t*)a.qa;
     const bf16_t* cache = (const bf16_t*)a.cache;
 
@@ -359,7 +369,7 @@ void latent_attn_mfma_kernel(AttnArgs a) {
         for (int ks = 0; ks < RV; ++ks) {
             const int r = 32 * ks + 8 * g;
             u32x4 v = {0u, 0u, 0u, 0u};
-            if (va && r < R) v = *(const u32x4*)(qr + r);
+            if (va && r < W) v = *(const u32x4*)(qr + r);
             qf[ks] = __builtin_bit_cast(bf16x8, v);
         }
     }
@@ -380,8 +390,9 @@ void latent_attn_mfma_kernel(AttnArgs a) {
     f32x4 oacc[NO];
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-        mrow[i] = -INFINITY;
-        lrow[i] = 0.f;
+        const bool snk = a.sink && valid_i[i] && a.parts == 1;
+        mrow[i] = snk ? a.sink[head_i[i]] : -INFINITY;
+        lrow[i] = snk ? 1.f : 0.f;
     }
 #pragma unroll
     for (int nt = 0; nt < NO; ++nt) oacc[nt] = (f32x4){0.f, 0.f, 0.f, 0.f};
@@ -393,7 +404,7 @@ void latent_attn_mfma_kernel(AttnArgs a) {
     // current tile's products and stay in registers meanwhile (all of a tile when NTH * UB covers it); the rest
     // is loaded UB pieces at a time once the tile's turn has come.
     const int bs_shift = (a.bs & (a.bs - 1)) == 0 ? __builtin_ctz(a.bs) : -1;
-    constexpr int CPK = RP / 8, TOTAL = KT * CPK, UB = (NW == 1 && RV > 8) || NW == 8 || (RS == 2 && RV > 12) ? 4 : 8;  // register room at the widest ranks
+    constexpr int CPK = RP / 8, TOTAL = KT * CPK, UB = NW == 8 && RV > 16 ? 5 : (NW == 1 && RV > 8) || NW == 8 || (RS == 2 && RV > 12) ? 4 : 8;  // register room at the widest ranks
     u32x4 pre[UB];
     auto fetch = [&](int k0, int base, u32x4* v) {
 #pragma unroll
@@ -402,11 +413,11 @@ void latent_attn_mfma_kernel(AttnArgs a) {
             const int p = id / CPK, c = id - p * CPK;
             const int key = k0 + p;
             v[u] = (u32x4){0u, 0u, 0u, 0u};
-            if (id < TOTAL && key < k_end && c * 8 < R) {
+            if (id < TOTAL && key < k_end && c * 8 < W) {
                 // block sizes are powers of two in practice: a shift instead of a division per piece
                 const int bi = bs_shift >= 0 ? key >> bs_shift : key / a.bs;
                 const int bo = key - bi * a.bs;
-                v[u] = *(const u32x4*)(cache + ((long)btr[bi] * a.bs + bo) * R + c * 8);
+                v[u] = *(const u32x4*)(cache + ((long)btr[bi] * a.bs + bo) * W + c * 8);
             }
         }
     };
@@ -532,35 +543,35 @@ void latent_attn_mfma_kernel(AttnArgs a) {
     }
 }
 
-template <int RV, int NW, int RS>
+template <int RV, int NVT, int NW, int RS>
 int launch_mfma(const AttnArgs& a, int n_rows, hipStream_t st) {
     constexpr int RP = RV * 32, BM = NW / RS * 16;
     constexpr size_t lds = (size_t)32 * (RP * 2 + 16) + (size_t)NW * 16 * (32 * 2 + 16);
     static_assert(lds <= 64 * 1024, "tile does not fit the LDS of a workgroup");
     const int tiles = a.cu_q ? (n_rows * a.H + BM - 1) / BM + a.n_seqs : a.n_seqs * ((a.H + BM - 1) / BM);
     dim3 grid(tiles, a.parts);
-    latent_attn_mfma_kernel<RV, NW, RS><<<grid, NW * 64, lds, st>>>(a);
+    latent_attn_mfma_kernel<RV, NVT, NW, RS><<<grid, NW * 64, lds, st>>>(a);
     return (int)hipGetLastError();
 }
 
-template <int RV>
+template <int RV, int NVT = RV * 2>
 int dispatch_mfma_nw(const AttnArgs& a, int n_rows, hipStream_t st) {
     // Row tiles per workgroup: prompt chunks four. A decode row set is one token's H heads: up to 16 take one row
     // tile, up to 32 two, more four. Ranks of 256 and more split each row tile between two waves (RS 2); narrower
     // ones keep one wave per row tile, with a second wave that only helps to fetch when there is a single row tile.
     const int rows = a.cu_q ? 64 : a.H;
     if constexpr (RV >= 8 && RV % 2 == 0) {
-        if (rows <= 16) return launch_mfma<RV, 2, 2>(a, n_rows, st);
-        if (rows <= 32) return launch_mfma<RV, 4, 2>(a, n_rows, st);
-        return launch_mfma<RV, 8, 2>(a, n_rows, st);
+        if (rows <= 16) return launch_mfma<RV, NVT, 2, 2>(a, n_rows, st);
+        if (rows <= 32) return launch_mfma<RV, NVT, 4, 2>(a, n_rows, st);
+        return launch_mfma<RV, NVT, 8, 2>(a, n_rows, st);
     } else {
-        if (rows <= 32) return launch_mfma<RV, 2, 1>(a, n_rows, st);
-        return launch_mfma<RV, 4, 1>(a, n_rows, st);
+        if (rows <= 32) return launch_mfma<RV, NVT, 2, 1>(a, n_rows, st);
+        return launch_mfma<RV, NVT, 4, 1>(a, n_rows, st);
     }
 }
 
 int dispatch_mfma(const AttnArgs& a, int n_rows, hipStream_t st) {
-    const int rv = (a.R + 31) / 32;
+    const int rv = (a.W + 31) / 32;
     if (rv <= 1) return dispatch_mfma_nw<1>(a, n_rows, st);
     if (rv <= 2) return dispatch_mfma_nw<2>(a, n_rows, st);
     if (rv <= 3) return dispatch_mfma_nw<3>(a, n_rows, st);
@@ -569,37 +580,40 @@ int dispatch_mfma(const AttnArgs& a, int n_rows, hipStream_t st) {
     if (rv <= 8) return dispatch_mfma_nw<8>(a, n_rows, st);
     if (rv <= 12) return dispatch_mfma_nw<12>(a, n_rows, st);
     if (rv <= 16) return dispatch_mfma_nw<16>(a, n_rows, st);
+    if (rv <= 18 && a.R <= 512) return dispatch_mfma_nw<18, 32>(a, n_rows, st);
+    if (rv <= 20) return dispatch_mfma_nw<20>(a, n_rows, st);
     return (int)hipErrorInvalidValue;
 }
 
 // the matrix-core kernel reads queries and latents in 16-byte pieces
 bool mfma_ok(const AttnArgs& a) {
-    return a.R % 8 == 0 && a.qs_t % 8 == 0 && a.qs_h % 8 == 0 && ((uintptr_t)a.qa & 15) == 0 &&
+    return a.W % 8 == 0 && a.qs_t % 8 == 0 && a.qs_h % 8 == 0 && ((uintptr_t)a.qa & 15) == 0 &&
            ((uintptr_t)a.cache & 15) == 0;
 }
 
 }  // namespace
 
-// qa / out element [token row * s_t + head * s_h + r]; cache [blocks][bs][R]; bt [n_seqs][bt_stride] block tables;
+// qa / out element [token row * s_t + head * s_h + r]; cache [blocks][bs][W], of which the first R numbers of a row are
+// the value (W = R: the whole row); sink: [H] extra scores in the denominator, or null; bt [n_seqs][bt_stride] block tables;
 // cu_q: chunk row offsets (relative to row_base) of n_seqs prompt chunks, or null for one row per sequence;
 // ctx: context length of each sequence including this step's rows; impl: 0 auto, 1 the VALU kernel; parts > 1 (decode only): every sequence's keys
 // are split into partitions of part_len and merged through part_ml [n_seqs * H * parts][2], part_o [..][R].
-extern "C" int mxl_latent_attn(const void* qa, long qs_t, long qs_h, const void* cache, int is16, int bs, int R,
-                               const int* bt, int bt_stride, const int* cu_q, const int* ctx, int n_seqs, int n_rows,
+extern "C" int mxl_latent_attn(const void* qa, long qs_t, long qs_h, const void* cache, int is16, int bs, int W,
+                               int R, const float* sink, const int* bt, int bt_stride, const int* cu_q, const int* ctx, int n_seqs, int n_rows,
                                int row_base, void* out, long os_t, long os_h, float scale, int H, int parts,
                                int part_len, float* part_ml, float* part_o, int impl, hipStream_t st) {
     if (n_seqs <= 0 || n_rows <= 0) return 0;
-    if (!(qa && cache && bt && ctx && out && bs > 0 && R > 0 && R <= 512 && H > 0 && bt_stride > 0 && parts >= 1))
+    if (!(qa && cache && bt && ctx && out && bs > 0 && R > 0 && W >= R && W <= 640 && H > 0 && bt_stride > 0 && parts >= 1))
         return (int)hipErrorInvalidValue;
     if (parts > 1 && (cu_q || !part_ml || !part_o || part_len <= 0 || parts > 1024)) return (int)hipErrorInvalidValue;
-    AttnArgs a{qa, qs_t, qs_h, cache, bs, R, bt, bt_stride, cu_q, ctx, n_seqs, row_base, out, os_t, os_h, scale,
-               H, parts, part_len, part_ml, part_o};
+    AttnArgs a{qa, qs_t, qs_h, cache, bs, W, R, bt, bt_stride, cu_q, ctx, n_seqs, row_base, out, os_t, os_h, scale,
+               H, parts, part_len, part_ml, part_o, sink};
     // impl 0: matrix cores where the layout allows (bf16, 16-byte pieces), else the fp32 VALU kernel; 1: VALU always
     int rc;
     if (is16 && impl == 0 && mfma_ok(a)) rc = dispatch_mfma(a, n_rows, st);
     else rc = is16 ? dispatch<true>(a, n_rows, st) : dispatch<false>(a, n_rows, st);
     if (rc != 0 || parts == 1) return rc;
-    if (is16) latent_attn_merge_kernel<true><<<n_seqs * H, 256, 0, st>>>(part_ml, part_o, parts, R, H, row_base, out, os_t, os_h);
-    else latent_attn_merge_kernel<false><<<n_seqs * H, 256, 0, st>>>(part_ml, part_o, parts, R, H, row_base, out, os_t, os_h);
+    if (is16) latent_attn_merge_kernel<true><<<n_seqs * H, 256, 0, st>>>(part_ml, part_o, parts, R, H, row_base, out, os_t, os_h, sink);
+    else latent_attn_merge_kernel<false><<<n_seqs * H, 256, 0, st>>>(part_ml, part_o, parts, R, H, row_base, out, os_t, os_h, sink);
     return (int)hipGetLastError();
 }

@@ -1,6 +1,7 @@
 // latent_ops.hip: the small fp32 row kernels of decoders built on ops/latent.py (scalar-gain RMS norm, embedding
 // gather + norm, sigmoid-gated normed residual add, squared ReLU, causal tap convolution with carried tails, the
-// two latent norms + paged append, per-head output gate + head-major -> token-major pack).
+// two latent norms + paged append, latent norm + rotary part + paged append beside the split of the queries, per-head or
+// per-number output gate + head-major -> token-major pack).
 //
 // All statistics, gates and the residual are fp32; 16-bit (bf16) appears only on outputs that feed a GEMM and in
 // the cached latent. Launchers are `extern "C" int mxl_*(..., hipStream_t)`, return the launch's hipError_t, never
@@ -299,14 +300,64 @@ __global__ __launch_bounds__(NT) void latent_norm_append_kernel(const float* y, 
     }
 }
 
+// Rows of a layer whose queries and keys have an unrotated and a rotated part: q heads of dim + rot numbers, one key row
+// of rank + rot numbers per token. grid (T, ceil((H + 1) / 4)), one wave per unit: unit h < H splits query head h (its
+// first dim numbers go to qn [T, H * dim], the rotated rest to columns rank .. of the absorbed query row (h, t) in qa);
+// unit H norms the latent (rank numbers, weight w) and appends it and the rotated key part as one cache row of
+// rank + rot numbers. Pair (2 i, 2 i + 1) of a rotated part turns by position * freqs[i]; both factors times mag.
+MX_DEV float turn_pair(const float* p, int e, float pos, const float* freqs, float mag) {
+    float s, c;
+    sincosf(pos * freqs[e >> 1], &s, &c);
+    const float u = p[e], v = p[e ^ 1];
+    return ((e & 1) ? u * c + v * s : u * c - v * s) * mag;
+}
+template <bool B16>
+__global__ __launch_bounds__(NT) void latent_rope_append_kernel(const float* q, int ldq, const float* kv, int ldkv, int H,
+                                                                int dim, int rot, int rank, const float* w, float eps,
+                                                                const float* freqs, float mag, const int* positions,
+                                                                void* qn, int ldqn, void* qa, long qs_t, long qs_h,
+                                                                void* cache, const int* slots) {
+    const int t = blockIdx.x, u = blockIdx.y * (NT / 64) + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+    const float pos = (float)positions[t];
+    if (u < H) {
+        const float* src = q + (long)t * ldq + (long)u * (dim + rot);
+        for (int e = lane; e < dim; e += 64) st_elem<B16>(qn, (long)t * ldqn + (long)u * dim + e, src[e]);
+        const long dst = (long)t * qs_t + (long)u * qs_h + rank;
+        for (int e = lane; e < rot; e += 64) st_elem<B16>(qa, dst + e, turn_pair(src + dim, e, pos, freqs, mag));
+        return;
+    }
+    if (u > H) return;
+    const int sl = slots[t];
+    if (sl < 0) return;
+    const float* src = kv + (long)t * ldkv;
+    const long dst = (long)sl * (rank + rot);
+    float keep[10], wk[10];  // ranks of up to 640 numbers stay in registers
+    float ss = 0.f;
+#pragma unroll
+    for (int k = 0; k < 10; ++k) {  // clamped addresses: straight-line loads, all in flight together
+        const int c = min(lane + k * 64, rank - 1);
+        keep[k] = lane + k * 64 < rank ? src[c] : 0.f;
+        wk[k] = w[c];
+        ss += keep[k] * keep[k];
+    }
+    const float sc = 1.f / sqrtf(wave_sum(ss) / (float)rank + eps);
+#pragma unroll
+    for (int k = 0; k < 10; ++k) {
+        const int c = lane + k * 64;
+        if (c < rank) st_elem<B16>(cache, dst + c, keep[k] * sc * wk[k]);
+    }
+    for (int e = lane; e < rot; e += 64) st_elem<B16>(cache, dst + rank + e, turn_pair(src + rank, e, pos, freqs, mag));
+}
+
+// per: numbers that share one gate (dv: one gate per head, 1: one per number)
 template <bool B16>
 __global__ __launch_bounds__(NT) void head_gate_pack_kernel(const float* ov, const float* gp, int ldg, void* out,
-                                                            int ldo, int H, int T, int dv) {
+                                                            int ldo, int H, int T, int dv, int per) {
     const int t = blockIdx.x;
     const int n = H * dv;
     for (int i = threadIdx.x; i < n; i += NT) {
         const int hh = i / dv, e = i - hh * dv;
-        const float v = ov[((long)hh * T + t) * dv + e] * sigmoidf_(gp[(long)t * ldg + hh]);
+        const float v = ov[((long)hh * T + t) * dv + e] * sigmoidf_(gp[(long)t * ldg + (per == 1 ? i : hh)]);
         st_elem<B16>(out, (long)t * ldo + i, v);
     }
 }
@@ -385,11 +436,29 @@ extern "C" int mxl_latent_norm_append(const float* y, int ldy, int q_rank, int r
     return (int)hipGetLastError();
 }
 
-extern "C" int mxl_head_gate_pack(const float* ov, const float* gp, int ldg, void* out, int ldo, int is16, int H, int T,
-                                  int dv, hipStream_t st) {
+extern "C" int mxl_latent_rope_append(const float* q, int ldq, const float* kv, int ldkv, int H, int dim, int rot,
+                                      int rank, const float* w, float eps, const float* freqs, float mag,
+                                      const int* positions, void* qn, int ldqn, void* qa, long qs_t, long qs_h,
+                                      int is16, void* cache, const int* slots, int T, hipStream_t st) {
     if (T <= 0) return 0;
-    MXL_CHECK(ov && gp && out && H > 0 && dv > 0 && ldg >= H && ldo >= H * dv);
-    if (is16) head_gate_pack_kernel<true><<<T, NT, 0, st>>>(ov, gp, ldg, out, ldo, H, T, dv);
-    else head_gate_pack_kernel<false><<<T, NT, 0, st>>>(ov, gp, ldg, out, ldo, H, T, dv);
+    MXL_CHECK(q && kv && w && positions && qn && qa && cache && slots && H > 0 && dim > 0 && rot >= 0 && rot % 2 == 0);
+    MXL_CHECK(rank > 0 && rank <= 640 && (rot == 0 || freqs) && ldq >= H * (dim + rot) && ldkv >= rank + rot &&
+              ldqn >= H * dim && H <= 65535);
+    const dim3 grid(T, (H + 1 + NT / 64 - 1) / (NT / 64));
+    if (is16)
+        latent_rope_append_kernel<true><<<grid, NT, 0, st>>>(q, ldq, kv, ldkv, H, dim, rot, rank, w, eps, freqs, mag,
+                                                             positions, qn, ldqn, qa, qs_t, qs_h, cache, slots);
+    else
+        latent_rope_append_kernel<false><<<grid, NT, 0, st>>>(q, ldq, kv, ldkv, H, dim, rot, rank, w, eps, freqs, mag,
+                                                              positions, qn, ldqn, qa, qs_t, qs_h, cache, slots);
+    return (int)hipGetLastError();
+}
+
+extern "C" int mxl_head_gate_pack(const float* ov, const float* gp, int ldg, void* out, int ldo, int is16, int H, int T,
+                                  int dv, int per, hipStream_t st) {
+    if (T <= 0) return 0;
+    MXL_CHECK(ov && gp && out && H > 0 && dv > 0 && ldo >= H * dv && (per == 1 || per == dv) && ldg >= H * dv / per);
+    if (is16) head_gate_pack_kernel<true><<<T, NT, 0, st>>>(ov, gp, ldg, out, ldo, H, T, dv, per);
+    else head_gate_pack_kernel<false><<<T, NT, 0, st>>>(ov, gp, ldg, out, ldo, H, T, dv, per);
     return (int)hipGetLastError();
 }

@@ -133,46 +133,53 @@ LATENT_SIGS = {
     "mxl_tap_conv": [P, I, P, I, P, P, P, I, P, I, P, I, I, I, I, P],
     # y, ldy, q_rank, rank, wq, wkv, eps, cq, ldcq, cq16, cache, cache16, slots, T, stream
     "mxl_latent_norm_append": [P, I, I, I, P, P, F, P, I, I, P, I, P, I, P],
-    # qa, qs_t, qs_h, cache, is16, bs, R, bt, bt_stride, cu_q, ctx, n_seqs, n_rows, row_base, out, os_t, os_h, scale,
+    # qa, qs_t, qs_h, cache, is16, bs, W, R, sink, bt, bt_stride, cu_q, ctx, n_seqs, n_rows, row_base, out, os_t, os_h, scale,
     # H, parts, part_len, part_ml, part_o, impl, stream
-    "mxl_latent_attn": [P, L, L, P, I, I, I, P, I, P, P, I, I, I, P, L, L, F, I, I, I, P, P, I, P],
-    # ov, gate_pre, ldg, out, ldo, is16, H, T, dv, stream
-    "mxl_head_gate_pack": [P, P, I, P, I, I, I, I, I, P],
+    "mxl_latent_attn": [P, L, L, P, I, I, I, I, P, P, I, P, P, I, I, I, P, L, L, F, I, I, I, P, P, I, P],
+    # q, ldq, kv, ldkv, H, dim, rot, rank, w, eps, freqs, mag, positions, qn, ldqn, qa, qs_t, qs_h, is16, cache, slots,
+    # T, stream
+    "mxl_latent_rope_append": [P, I, P, I, I, I, I, I, P, F, P, F, P, P, I, P, L, L, I, P, P, I, P],
+    # ov, gate_pre, ldg, out, ldo, is16, H, T, dv, numbers per gate, stream
+    "mxl_head_gate_pack": [P, P, I, P, I, I, I, I, I, I, P],
 }
 
 # libmxh.so (csrc/kernels/hybrid/): kernels of the hybrid attention / recurrent decoders (ops/hybrid.py)
 HYBRID_SIGS = {
-    # table, is16, V, tokens, out, ldo, accumulate, out16, ld16, T, C, stream
-    "mxh_embed_rows": [P, I, I, P, P, I, I, P, I, I, I, P],
+    # table, is16, V, tokens, out, ldo, accumulate, out16, ld16, scale, T, C, stream
+    "mxh_embed_rows": [P, I, I, P, P, I, I, P, I, F, I, I, P],
     # x, ldx, rows, w, offset, eps, out32, ld32, out16, ld16, M, C, stream
     "mxh_offset_norm": [P, I, P, P, F, F, P, I, P, I, I, I, P],
     # y, ldy, w, offset, eps, x, ldx, out16, ld16, T, C, stream
     "mxh_norm_add": [P, I, P, F, F, P, I, P, I, I, I, P],
+    # y, ldy, bias, scale, x, ldx, norm_w, offset, eps, out32, ld32, out16, ld16, T, C, stream
+    "mxh_scale_add_norm": [P, I, P, P, P, I, P, F, F, P, I, P, I, I, I, P],
     # q, k, v, ldq, ldk, ldv, positions, H, G, dk, dv, rot_dims, base, norm, eps, q_out, ldqo, q16, kc, vc, c16, slots,
     # q_weight, k_weight, temp_coef, temp_every, T, stream
-    # ..., temp_every, half, value heads, T, stream
-    "mxh_rope_norm_append": [P, P, P, I, I, I, P, I, I, I, I, I, F, I, F, P, I, I, P, P, I, P, P, P, F, I, I, I, I, P],
+    # ..., temp_every, half, value heads, freqs, mag, q_bias, k_bias, v_bias, T, stream
+    "mxh_rope_norm_append": [P, P, P, I, I, I, P, I, I, I, I, I, F, I, F, P, I, I, P, P, I, P, P, P, F, I, I, I, P, F, P,
+                             P, P, I, P],
     # q, ldq, q16, kc, vc, bs, bt, bt_stride, cu_q, ctx, n_seqs, n_rows, row_base, out, ldo, o16, H, G, dk, dv, scale,
     # chunk, window, sink, out_scale, row_off, parts, part_len, part_ml, part_o, sink_v, bias, bias_rows, gate, ldg,
     # stream
-    # (value heads before the stream)
+    # (value heads and kept first tokens before the stream)
     "mxh_attention": [P, I, I, P, P, I, P, I, P, P, I, I, I, P, I, I, I, I, I, I, F, I, I, I, F, I, I, I, P, P, P, P, I,
-                      P, I, I, P],
+                      P, I, I, I, P],
     # q, ldq, kc, vc, bs, table, p0, n, out, ldo, o16, H, G, dk, dv, scale, chunk, window, sink, out_scale, sink_v,
     # bias, bias_rows, gate, ldg, stream
-    # (value heads and the two-part weights flag before the stream)
-    "mxh_attention_mfma": [P, I, P, P, I, P, I, I, P, I, I, I, I, I, I, F, I, I, I, F, P, P, I, P, I, I, I, P],
+    # (value heads, the two-part weights flag and the kept first tokens before the stream)
+    "mxh_attention_mfma": [P, I, P, P, I, P, I, I, P, I, I, I, I, I, I, F, I, I, I, F, P, P, I, P, I, I, I, I, P],
     "mxh_attention_mfma_ok": [I, I],
     # q, ldq, kc, vc, bs, bt, bt_stride, ctx, n_seqs, out, ldo, o16, H, G, dk, dv, scale, chunk, window, sink, out_scale,
     # parts, part_len, part_ml, part_o, sink_v, bias, bias_rows, gate, ldg, stream
     "mxh_attention_decode_mfma": [P, I, P, P, I, P, I, P, I, P, I, I, I, I, I, I, F, I, I, I, F, I, I, P, P, P, P, I, P,
-                                  I, I, I, P],
-    # kc, vc, is16, bs, table, lo, n, G, dk, dv, kh, vh, stream
-    "mxh_kv_gather": [P, P, I, I, P, I, I, I, I, I, P, P, I, P],
+                                  I, I, I, I, P],
+    # kc, vc, is16, bs, table, lo, n, G, dk, dv, kh, vh, value heads, kept first tokens, stream
+    "mxh_kv_gather": [P, P, I, I, P, I, I, I, I, I, P, P, I, I, P],
     # src, s16, s_stride_i, s_stride_h, dst, d16, d_stride_i, d_stride_h, n, H, d, scale, gate, ldg, stream
     "mxh_head_transpose": [P, I, L, L, P, I, L, L, I, I, I, F, P, I, P],
-    # scores, weights, w16, rows, n, nk, p0, key0, scale, chunk, window, sink, sink_v, bias, bias_rows, H, stream
-    "mxh_masked_softmax": [P, P, I, L, I, I, I, I, F, I, I, I, P, P, I, I, I, P],
+    # scores, weights, w16, rows, n, nk, p0, key0, scale, chunk, window, sink, sink_v, bias, bias_rows, H, two,
+    # columns of kept first tokens, kept first tokens, stream
+    "mxh_masked_softmax": [P, P, I, L, I, I, I, I, F, I, I, I, P, P, I, I, I, I, I, P],
     # x, ldx, w, bias, taps, silu, tails, state, positions, n_dec, pf_cu, n_pf, out, ldo, T, C, stream
     "mxh_causal_conv": [P, I, P, P, I, I, P, P, P, I, P, I, P, I, I, I, P],
     # x, ldx, heads, dim, eps, scale, split, scale2, T, stream
@@ -186,10 +193,11 @@ HYBRID_SIGS = {
     "mxh_state_scan": [P, I, P, I, P, I, P, I, P, I, I, P, P, P, P, I, P, I, P, I, I, I, I, I, I, I, F, P],
     # y, ldy, gate, ldg, w, wlen, eps, group, gate_first, out_scale, out, ldo, o16, T, C, sigmoid gate, proj, R, stream
     "mxh_gated_group_norm": [P, I, P, I, P, I, F, I, I, F, P, I, I, I, I, I, P, I, P],
-    # a, lda, b, ldb, bias_a, bias_b, scale, lds, group, scale_sigmoid, out, ldo, o16, T, F, act, stream
-    "mxh_glu": [P, I, P, I, P, P, P, I, I, I, P, I, I, I, I, I, P],
-    # logits, ld, bias, T, E, top, scale, eps, weights, sigmoid scores, stream
-    "mxh_moe_route": [P, I, P, I, I, I, F, F, P, I, P],
+    # a, lda, b, ldb, bias_a, bias_b, scale, lds, group, scale_sigmoid, out, ldo, o16, T, F, act, limit, alpha,
+    # stream
+    "mxh_glu": [P, I, P, I, P, P, P, I, I, I, P, I, I, I, I, I, F, F, P],
+    # logits, ld, bias, T, E, top, scale, eps, weights, mode, groups, groups kept, stream
+    "mxh_moe_route": [P, I, P, I, I, I, F, F, P, I, I, I, P],
     # table, pair, is16, V, tokens, seq_state, positions, n_dec, pf_cu, n_pf, last, scale, mul_prev, mul_cur, buckets,
     # out, copies, T, C, stream
     "mxh_embed_pair": [P, P, I, I, P, P, P, I, P, I, P, F, I, I, I, P, I, I, I, P],

@@ -383,14 +383,16 @@ class LLMEngine:
         # paged-pool-plus-state models: a paged pool addressed like K / V blocks (per-token latents, models/vosotar.py;
         # keys and values of the attention layers of a hybrid decoder, models/vugotar.py) plus one state slot per live
         # sequence (SlotPool) for what is carried between steps (convolution tails, recurrent states). A cached block
-        # does not hold that carried state, so blocks are not shared between requests; no drafts, no TP
+        # does not hold that carried state, so blocks are not shared between requests unless the model says that its
+        # pages hold everything a sequence carries (`pages_only`, models/zomolix.py); no drafts, no TP
         self.latent = getattr(model, "cache_kind", "") in ("latent", "hybrid")
         self.state_slots = None
         self._replay: dict = {}
         if self.latent:
             if tp is not None:
                 raise ValueError("tensor parallelism is not supported for latent-cache models")
-            c.enable_prefix_cache = False
+            if not getattr(model, "pages_only", False):
+                c.enable_prefix_cache = False
             draft = None
         self.max_blocks_per_seq = (c.max_model_len + c.block_size - 1) // c.block_size
         use_spec = draft is not None and c.n_draft > 0 and tp is None

@@ -213,11 +213,13 @@ class HybridCache:
     * `kv[i]`: (keys [num_blocks, block_size, kv_heads * dim], values [.., kv_heads * vdim]) in bf16 or fp32,
       token-major so one append writes one contiguous row, addressed by the block tables and flat slots of the block
       manager; None for runs without attention;
+    * `lat[i]`: [num_blocks, block_size, row] in bf16 or fp32, one row per token that serves as key and value of every
+      head (ops/latent.py: a latent, with a rotated key part beside it), addressed the same way; None otherwise;
     * `state[i]`: fp32 [state_slots, heads, P, N] recurrent state (N numbers for each of a head's P value columns),
       None for runs without a recurrence;
     * `tails[i]`: fp32 [state_slots, taps - 1, channels] last inputs of the run's causal convolution, or None.
 
-    `spec` lists per run a dict with the optional keys "kv": (key row, value row), "state": (heads, P, N),
+    `spec` lists per run a dict with the optional keys "kv": (key row, value row), "lat": row, "state": (heads, P, N),
     "tails": (taps - 1, channels). State slots are handed out per live sequence by `SlotPool`. With `seq_tokens` the
     cache also carries `last_token` int32 [state_slots]: the newest token of each live sequence, for embeddings that
     look at the token before."""
@@ -229,8 +231,11 @@ class HybridCache:
         S = max(1, state_slots)
         f32 = dict(dtype=torch.float32, device=device)
         self.last_token = torch.zeros(S, dtype=torch.int32, device=device) if seq_tokens else None
-        self.kv, self.state, self.tails = [], [], []
+        self.kv, self.lat, self.state, self.tails = [], [], [], []
         for e in spec:
+            row = e.get("lat")
+            self.lat.append(None if row is None else
+                            torch.zeros((num_blocks, block_size, int(row)), dtype=dtype, device=device))
             kv, st, tl = e.get("kv"), e.get("state"), e.get("tails")
             self.kv.append(None if kv is None else
                            (torch.zeros((num_blocks, block_size, int(kv[0])), dtype=dtype, device=device),
@@ -240,6 +245,11 @@ class HybridCache:
 
     def layer(self, i: int):
         return self.kv[i], self.state[i], self.tails[i]
+
+    @staticmethod
+    def pool_numbers(spec) -> list:
+        """Numbers per token of every run that keeps something per token (what one block's bytes are counted from)."""
+        return [sum(e.get("kv") or ()) + int(e.get("lat") or 0) for e in spec if e.get("kv") or e.get("lat")]
 
     def state_bytes_per_seq(self) -> int:
         return int(sum(t[0].numel() * 4 for t in self.state + self.tails if t is not None))

@@ -205,16 +205,11 @@ class VosotarModel:
     tp_size = 1
     n_kv = 1
     n_heads = 1
-    DECODE_WGS = 512  # decode attention: workgroups to aim for when splitting contexts into key partitions
+    DECODE_WGS = LA.DECODE_WGS  # decode attention: workgroups to aim for when splitting contexts into key partitions
 
     def decode_part_len(self, n_dec: int, heads: int, max_len: int) -> int:
-        """Keys per partition of the decode attention: a workgroup holds up to 64 (token, head) rows of one
-        sequence, so few sequences with long contexts are split finely (down to one 32-key tile) to cover the CUs, and
-        large batches coarsely (fewer partials to merge)."""
-        wgs = max(1, n_dec * -(-heads // (32 if heads <= 32 else 64)))
-        want = max(1, self.DECODE_WGS // wgs)  # partitions per sequence
-        per = -(-max(1, max_len) // want)
-        return max(32, -(-per // 32) * 32)
+        """Keys per partition of the decode attention (ops/latent.py decode_part_len)."""
+        return LA.decode_part_len(n_dec, heads, max_len, self.DECODE_WGS)
 
     def __init__(self, cfg: VosotarConfig, device="cpu", dtype=None):
         self.cfg = cfg

@@ -3,11 +3,13 @@
 * `embed_rows`, `offset_rmsnorm`, `norm_add`: an fp32 residual from a 16-bit table; an RMS norm whose weight is
   stored around an offset (x / rms * (offset + w)); the same norm applied to a sublayer's OUTPUT and added to the
   residual (x += y / rms(y) * (offset + w)), with the 16-bit copy of the new residual the next GEMM reads;
-* `rope_norm_append`: rotary positions on neighbouring pairs of the first `rot_dims` numbers of each query / key
-  head, an optional unit-RMS norm of every head after the rotation (with optional per-channel weights), an optional
+* `scale_add_norm`: x += (y + bias) * s with one factor per column (layer scale) and, in the same pass, the norm of the
+  new residual that the next sublayer reads;
+* `rope_norm_append`: projection biases, rotary positions on neighbouring pairs (or half pairs) of the first `rot_dims`
+  numbers of each query / key head, by base^(-2i/d) or by given frequencies with a magnitude (scaled rotations), an optional unit-RMS norm of every head after the rotation (with optional per-channel weights), an optional
   position-dependent query temperature, and the append of keys and values to paged pools;
 * `masked_attention`: causal attention over the paged pools whose visible range starts at a chunk border
-  (`chunk`), `window` keys back, or at position 0, with an optional sink (one extra term exp(0), or exp(s_h) with a
+  (`chunk`), `window` keys back (with the first `keep` tokens still visible), or at position 0, with an optional sink (one extra term exp(0), or exp(s_h) with a
   learned s_h per head, in the softmax denominator that carries no value), an optional additive bias that depends on
   the distance between query and key (`log_bucket_table`) and an optional sigmoid gate per token and head;
 * `causal_conv`: a per-channel causal convolution over time (optional bias and SiLU) whose last taps-1 inputs are
@@ -18,11 +20,13 @@
   optional skip D v on the output (state-space duality form); the decay a is one number per head or, for gated
   linear attention, one per key channel (S <- diag(a) S + k v^T, a = sigmoid(z)^(1/tau));
 * `gated_group_norm`: unit-RMS norm over groups of columns, a weight, and a SiLU gate before or after the norm;
-* `glu`: silu(a + bias) * (b + bias) with an optional per-row, per-column-group factor (routing weights of experts
+* `glu`: silu(a + bias) * (b + bias), or other gated units (tanh gelu, squared ReLU, a clamped sigmoid unit), with an
+  optional per-row, per-column-group factor (routing weights of experts
   evaluated side by side, or the sigmoid gate of a shared expert);
 * `moe_route`: softmax over experts (optional logit bias), the `top` largest, renormalised and scaled, as a dense
   [T, E] weight matrix (with eps = 0 and scale = 1 that is the softmax over the chosen logits alone); or, in the
-  `sigmoid` mode, the chosen experts' sigmoid scores as they are;
+  `sigmoid` / `scores` modes, the chosen experts' sigmoid / softmax scores as they are; optionally only from the best
+  groups of neighbouring experts;
 * `embed_pair`: a scaled token embedding plus a row of a second table picked by a hash of (previous token, token); the
   previous token is carried per sequence;
 * `hyper_step`: a residual kept as several streams: the streams are mixed among themselves and take a sublayer's
@@ -52,21 +56,21 @@ def _f32c(t: torch.Tensor, what: str):
 
 # ------------------------------------------------------------------------------------------------ embedding, norm
 def embed_rows(table: torch.Tensor, tokens: torch.Tensor, out: torch.Tensor, accumulate: bool = False,
-               out16: torch.Tensor | None = None):
-    """out[t] (=|+=) table[tokens[t]]; table fp32 or bf16 [V, C], out fp32 [T, C]; `out16` (bf16 [T, C]) also receives
+               out16: torch.Tensor | None = None, scale: float = 1.0):
+    """out[t] (=|+=) scale * table[tokens[t]]; table fp32 or bf16 [V, C], out fp32 [T, C]; `out16` (bf16 [T, C]) also receives
     the result, rounded (the operand of a GEMM that reads the residual itself)."""
     T, C = out.shape
     if T == 0:
         return out
     if not out.is_cuda:
-        rows = table[tokens.long()].float()
+        rows = table[tokens.long()].float() * scale
         out.add_(rows) if accumulate else out.copy_(rows)
         if out16 is not None:
             out16.copy_(out)
         return out
     N.kcall("mxh_embed_rows", table.data_ptr(), _is16(table), table.shape[0], tokens.data_ptr(), out.data_ptr(),
-            out.stride(0), int(accumulate), N.ptr(out16), out16.stride(0) if out16 is not None else 0, T, C,
-            N.stream_ptr())
+            out.stride(0), int(accumulate), N.ptr(out16), out16.stride(0) if out16 is not None else 0, float(scale), T,
+            C, N.stream_ptr())
     return out
 
 
@@ -109,6 +113,34 @@ def norm_add(y: torch.Tensor, w: torch.Tensor, eps: float, x: torch.Tensor, out1
     _f32c(x, "norm_add")
     N.kcall("mxh_norm_add", y.data_ptr(), y.stride(0), w.data_ptr(), float(offset), float(eps), x.data_ptr(),
             x.stride(0), N.ptr(out16), out16.stride(0) if out16 is not None else 0, T, C, N.stream_ptr())
+    return x
+
+
+def scale_add_norm(y: torch.Tensor, bias: torch.Tensor | None, scale: torch.Tensor | None, x: torch.Tensor,
+                   norm_w: torch.Tensor | None = None, eps: float = 0.0, out32: torch.Tensor | None = None,
+                   out16: torch.Tensor | None = None, offset: float = 0.0):
+    """x += (y + bias) * scale on fp32 rows [T, C] (bias, scale fp32 [C]; None: 0 and 1): a sublayer's output enters the
+    residual through a layer scale. With `norm_w` the same pass writes the norm the next sublayer reads,
+    x / sqrt(mean(x^2) + eps) * (offset + norm_w) of the new x, as fp32 (`out32`) and / or bf16 (`out16`)."""
+    T, C = y.shape
+    if T == 0:
+        return x
+    if norm_w is not None and out32 is None and out16 is None:
+        raise ValueError("scale_add_norm: a norm needs an output")
+    if not y.is_cuda:
+        z = y if bias is None else y + bias
+        x.add_(z if scale is None else z * scale)
+        if norm_w is not None:
+            offset_rmsnorm(x, norm_w, eps, out32, out16, offset=offset)
+        return x
+    _f32c(y, "scale_add_norm")
+    _f32c(x, "scale_add_norm")
+    for v in (bias, scale, norm_w):
+        if v is not None and (v.dtype != torch.float32 or v.numel() != C or not v.is_contiguous()):
+            raise TypeError("scale_add_norm: fp32 vectors of one number per column")
+    N.kcall("mxh_scale_add_norm", y.data_ptr(), y.stride(0), N.ptr(bias), N.ptr(scale), x.data_ptr(), x.stride(0),
+            N.ptr(norm_w), float(offset), float(eps), N.ptr(out32), out32.stride(0) if out32 is not None else 0,
+            N.ptr(out16), out16.stride(0) if out16 is not None else 0, T, C, N.stream_ptr())
     return x
 
 
@@ -220,7 +252,9 @@ def rope_norm_append(q_in: torch.Tensor, k_in: torch.Tensor, v_in: torch.Tensor,
                      G: int, dk: int, dv: int, rot_dims: int, rot_base: float, norm: bool, eps: float,
                      q_out: torch.Tensor, kc: torch.Tensor | None, vc: torch.Tensor | None, slots: torch.Tensor,
                      q_weight: torch.Tensor | None = None, k_weight: torch.Tensor | None = None, q_temp=None,
-                     half: bool = False, v_heads: int | None = None):
+                     half: bool = False, v_heads: int | None = None, freqs: torch.Tensor | None = None, mag: float = 1.0,
+                     q_bias: torch.Tensor | None = None, k_bias: torch.Tensor | None = None,
+                     v_bias: torch.Tensor | None = None):
     """q_in [T, H*dk], k_in [T, G*dk], v_in [T, Gv*dv] (Gv = v_heads, G when not given: the value pool may hold fewer
     heads than the key pool): fp32 column slices of one projection output. Pair (2i, 2i+1), or with `half` the pair
     (i, i + rot_dims/2), of a head's first rot_dims numbers turns by positions[t] * rot_base^(-2i / rot_dims); with
@@ -229,22 +263,30 @@ def rope_norm_append(q_in: torch.Tensor, k_in: torch.Tensor, v_in: torch.Tensor,
     (fp32 [dk], shared by the heads) when given. `q_temp` = (coef, every) multiplies the query at position p by
     1 + coef * ln(floor((p + 1) / every) + 1). Queries go to q_out [T, H*dk] (fp32 or bf16), keys and values into the
     paged pools kc [blocks, bs, G*dk] / vc [blocks, bs, G*dv] at flat slot slots[t] (slot < 0: not stored). With
-    k_in = None only the queries are made (a layer that reads another layer's keys and values)."""
+    k_in = None only the queries are made (a layer that reads another layer's keys and values). `q_bias`, `k_bias`,
+    `v_bias` (fp32, one number per column) are added first. `freqs` (fp32 [rot_dims / 2]) replaces the angles per
+    position, pair i turns by positions[t] * freqs[i]; sine and cosine are multiplied by `mag`."""
     T = q_in.shape[0]
     if T == 0:
         return
     if rot_dims % 2 or rot_dims > dk:
         raise ValueError("rope_norm_append: rot_dims is even and at most the head size")
     Gv = G if v_heads is None else int(v_heads)
+    if freqs is not None and (freqs.dtype != torch.float32 or freqs.numel() != rot_dims // 2):
+        raise TypeError("rope_norm_append: one fp32 frequency per pair")
+    for b_, n_ in ((q_bias, H * dk), (k_bias, G * dk), (v_bias, Gv * dv)):
+        if b_ is not None and (b_.dtype != torch.float32 or b_.numel() != n_ or not b_.is_contiguous()):
+            raise TypeError("rope_norm_append: fp32 biases of one number per column")
     if not q_in.is_cuda:
-        def turn(x, n, w=None):
-            x = _rope_ref(x.float().reshape(T, n, dk), positions, rot_dims, rot_base, half)
+        def turn(x, n, w=None, b=None):
+            x = x.float() if b is None else x.float() + b
+            x = _rope_ref(x.reshape(T, n, dk), positions, rot_dims, rot_base, half, freqs, mag)
             if norm:
                 x = x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps)
                 if w is not None:
                     x = x * w.float()
             return x.reshape(T, n * dk)
-        qn = turn(q_in, H, q_weight)
+        qn = turn(q_in, H, q_weight, q_bias)
         if q_temp is not None:
             coef, every = float(q_temp[0]), int(q_temp[1])
             qn = qn * (1.0 + coef * torch.log((torch.div(positions + 1, every, rounding_mode="floor") + 1).float()))[:, None]
@@ -252,8 +294,9 @@ def rope_norm_append(q_in: torch.Tensor, k_in: torch.Tensor, v_in: torch.Tensor,
         if k_in is None:
             return
         ok = slots >= 0
-        kc.view(-1, G * dk)[slots[ok].long()] = turn(k_in, G, k_weight)[ok].to(kc.dtype)
-        vc.view(-1, Gv * dv)[slots[ok].long()] = v_in.float()[ok].to(vc.dtype)
+        kc.view(-1, G * dk)[slots[ok].long()] = turn(k_in, G, k_weight, k_bias)[ok].to(kc.dtype)
+        v = v_in.float() if v_bias is None else v_in.float() + v_bias
+        vc.view(-1, Gv * dv)[slots[ok].long()] = v[ok].to(vc.dtype)
         return
     if (q_weight is not None or k_weight is not None) and not norm:
         raise ValueError("rope_norm_append: head weights belong to the head norm")
@@ -272,17 +315,20 @@ def rope_norm_append(q_in: torch.Tensor, k_in: torch.Tensor, v_in: torch.Tensor,
     N.kcall("mxh_rope_norm_append", q_in.data_ptr(), k_in.data_ptr(), v_in.data_ptr(), q_in.stride(0),
             k_in.stride(0), v_in.stride(0), positions.data_ptr(), H, G, dk, dv, rot_dims, float(rot_base), int(norm),
             float(eps), q_out.data_ptr(), q_out.stride(0), _is16(q_out), kc.data_ptr(), vc.data_ptr(), _is16(kc),
-            slots.data_ptr(), N.ptr(q_weight), N.ptr(k_weight), coef, every, int(half), Gv, T, N.stream_ptr())
+            slots.data_ptr(), N.ptr(q_weight), N.ptr(k_weight), coef, every, int(half), Gv, N.ptr(freqs),
+            float(mag), N.ptr(q_bias), N.ptr(k_bias), N.ptr(v_bias), T, N.stream_ptr())
 
 
-def _rope_ref(x: torch.Tensor, positions: torch.Tensor, rot_dims: int, rot_base: float, half: bool) -> torch.Tensor:
+def _rope_ref(x: torch.Tensor, positions: torch.Tensor, rot_dims: int, rot_base: float, half: bool, freqs=None,
+              mag: float = 1.0) -> torch.Tensor:
     """x fp32 [T, n, d]: a copy whose first rot_dims numbers per head are turned by the rows' positions."""
     x = x.clone()
     if rot_dims:
         n2 = rot_dims // 2
-        i = torch.arange(n2, dtype=torch.float32)
-        a = positions.float()[:, None] * torch.exp(i * (-2.0 / rot_dims * math.log(rot_base)))[None, :]
-        c, s = torch.cos(a)[:, None, :], torch.sin(a)[:, None, :]
+        if freqs is None:
+            freqs = torch.exp(torch.arange(n2, dtype=torch.float32) * (-2.0 / rot_dims * math.log(rot_base)))
+        a = positions.float()[:, None] * freqs[None, :]
+        c, s = torch.cos(a)[:, None, :] * mag, torch.sin(a)[:, None, :] * mag
         lo, hi = (slice(0, n2), slice(n2, rot_dims)) if half else (slice(0, rot_dims, 2), slice(1, rot_dims, 2))
         u, v = x[..., lo].clone(), x[..., hi].clone()
         x[..., lo] = u * c - v * s
@@ -316,7 +362,7 @@ def rope_rows(x: torch.Tensor, positions: torch.Tensor, heads: int, dim: int, ro
 
 
 def _attn_ref(q, kc, vc, table, ctx, pos0, H, G, dk, dv, scale, chunk, window, sink, out, out_scale, sink_v=None,
-              bias=None, gate=None, Gv=None):
+              bias=None, gate=None, Gv=None, keep=0):
     bs = kc.shape[1]
     nb = -(-ctx // bs)
     k = kc[table[:nb].long()].reshape(nb * bs, G, dk)[:ctx].float()
@@ -331,7 +377,7 @@ def _attn_ref(q, kc, vc, table, ctx, pos0, H, G, dk, dv, scale, chunk, window, s
     i = pos0 + torch.arange(n)[:, None]
     j = torch.arange(ctx)[None, :]
     lo = (i // chunk) * chunk if chunk else (i - window + 1).clamp(min=0) if window else torch.zeros_like(i)
-    vis = (j <= i) & (j >= lo)
+    vis = (j <= i) & ((j >= lo) | (j < keep))
     if bias is not None:
         s = s + bias.float()[:, (i - j).clamp(0, bias.shape[1] - 1)]
     s = s.masked_fill(~vis[None], float("-inf"))
@@ -374,6 +420,8 @@ def _visible_blocks(p0: int, n: int, chunk: int, window: int, heads: int):
     for a, b, key0 in spans:
         k0 = key0 if key0 is not None else 0
         rows = max(GEMM_MIN_ROWS, GEMM_MAX_SCORES // max(1, heads * (b - k0)))
+        if window:  # a block's keys reach a window behind its first row: blocks of about that size waste little
+            rows = min(rows, max(256, window))
         for a2 in range(a, b, rows):
             b2 = min(b, a2 + rows)
             out.append((a2, b2, key0 if key0 is not None else max(0, a2 - window + 1) if window else 0))
@@ -381,9 +429,9 @@ def _visible_blocks(p0: int, n: int, chunk: int, window: int, heads: int):
 
 
 def _attn_gemm_chunk(q, kc, vc, table, p0, n, H, G, dk, dv, scale, chunk, window, sink, out, out_scale, sink_v=None,
-                     bias=None, gate=None, Gv=None, p32=False):
+                     bias=None, gate=None, Gv=None, p32=False, keep=0):
     """A long prompt chunk (rows q [n, H*dk] at positions p0 ..) as library GEMMs: per block of rows, the visible keys
-    and values are gathered head-major from the pages, scores = Q K^T (fp32), masked sink softmax, out = P V (fp32).
+    and values (with a window also the `keep` first tokens) are gathered head-major from the pages, scores = Q K^T (fp32), masked sink softmax, out = P V (fp32).
     With `p32` and bf16 operands every softmax weight is written as two bf16 numbers (its rounding and the rest), side
     by side along K, and the values are stacked twice: the product sees the weights to 16 bits of mantissa."""
     from .dense import bmm_f32
@@ -391,21 +439,22 @@ def _attn_gemm_chunk(q, kc, vc, table, p0, n, H, G, dk, dv, scale, chunk, window
     md, dev, rep, bs = q.dtype, q.device, H // G, kc.shape[1]
     i16 = _is16(q)
     for a, b, key0 in _visible_blocks(p0, n, chunk, window, H):
-        n2, nk = b - a, b - key0
+        kn = min(keep, key0) if window else 0
+        n2, nk = b - a, b - key0 + kn
         kh = torch.empty((G, nk, dk), dtype=md, device=dev)
         vh = torch.empty((G, nk, dv), dtype=md, device=dev)
         N.kcall("mxh_kv_gather", kc.data_ptr(), vc.data_ptr(), i16, bs, table.data_ptr(), key0, nk, G, dk, dv,
-                kh.data_ptr(), vh.data_ptr(), G if Gv is None else Gv, st)
+                kh.data_ptr(), vh.data_ptr(), G if Gv is None else Gv, kn, st)
         qh = torch.empty((H, n2, dk), dtype=md, device=dev)
         qr = q[a - p0:]
         N.kcall("mxh_head_transpose", qr.data_ptr(), i16, qr.stride(0), dk, qh.data_ptr(), i16, dk, n2 * dk, n2, H, dk,
                 1.0, None, 0, st)
-        sc = bmm_f32(qh.view(G, rep * n2, dk), kh.transpose(1, 2))
+        sc = bmm_f32(qh.view(G, rep * n2, dk), kh.transpose(1, 2).contiguous())
         two = bool(p32 and i16)
         pw = torch.empty((G, rep * n2, 2 * nk if two else nk), dtype=md, device=dev)
         N.kcall("mxh_masked_softmax", sc.data_ptr(), pw.data_ptr(), i16, H * n2, n2, nk, a, key0, float(scale),
                 int(chunk), int(window), int(sink), N.ptr(sink_v), N.ptr(bias), bias.shape[1] if bias is not None else 0,
-                H, int(two), st)
+                H, int(two), kn, int(keep), st)
         o = bmm_f32(pw, torch.cat([vh, vh], 1) if two else vh)
         orow = out[a - p0:]
         grow = gate[a - p0:] if gate is not None else None
@@ -416,13 +465,14 @@ def _attn_gemm_chunk(q, kc, vc, table, p0, n, H, G, dk, dv, scale, chunk, window
 def masked_attention(q: torch.Tensor, kc: torch.Tensor, vc: torch.Tensor, rag: Ragged, H: int, G: int, dk: int, dv: int,
                      scale: float, out: torch.Tensor, chunk: int = 0, window: int = 0, sink=False,
                      out_scale: float = 1.0, workspace=None, bias: torch.Tensor | None = None,
-                     gate: torch.Tensor | None = None, v_heads: int | None = None, p32: bool = False):
+                     gate: torch.Tensor | None = None, v_heads: int | None = None, p32: bool = False, keep: int = 0):
     """Causal attention of q [T, H*dk] over the paged pools (rope_norm_append's layout); query head h reads key
     head g = h // (H / G) and value head g % v_heads (v_heads = G when not given; fewer value heads than key heads:
     several attention maps over the same values). `p32`: softmax weights enter the value product with more than
     bf16's mantissa also in bf16 mode (the row kernels keep them in fp32 anyway; the matrix-core kernels and the GEMM
     route split each weight into two bf16 numbers, its rounding and the rounding of the rest). The row at position i
-    sees j in [lo, i]: lo = (i // chunk) * chunk with `chunk`, max(0, i - window + 1) with `window`, else 0. `sink` = True adds exp(0) to the softmax denominator, an fp32 tensor
+    sees j in [lo, i]: lo = (i // chunk) * chunk with `chunk`, max(0, i - window + 1) with `window`, else 0; with a
+    window the positions below `keep` stay visible as well, at their true distance. `sink` = True adds exp(0) to the softmax denominator, an fp32 tensor
     [H] adds exp(sink[h]). `bias` (fp32 [H, L], contiguous) adds bias[h, min(i - j, L - 1)] to the scaled score.
     `gate` (fp32 [T, H], may be a column slice) multiplies head h's output of row t by sigmoid(gate[t, h]). out
     [T, H*dv] (may be a column slice; fp32 or bf16) receives out_scale times the result. q, pools and out share fp32
@@ -441,6 +491,8 @@ def masked_attention(q: torch.Tensor, kc: torch.Tensor, vc: torch.Tensor, rag: R
     Gv = G if v_heads is None else int(v_heads)
     if Gv < 1 or G % Gv:
         raise ValueError("masked_attention: the key heads are a multiple of the value heads")
+    if keep < 0 or (keep and (chunk or not window)):
+        raise ValueError("masked_attention: first tokens are kept in front of a window")
     sink_v = sink if isinstance(sink, torch.Tensor) else None
     sink = sink_v is not None or bool(sink)
     if sink_v is not None and (sink_v.dtype != torch.float32 or sink_v.numel() != H or not sink_v.is_contiguous()):
@@ -456,7 +508,7 @@ def masked_attention(q: torch.Tensor, kc: torch.Tensor, vc: torch.Tensor, rag: R
             lens = rag.dec_lens.tolist()
             for i in range(nd):
                 _attn_ref(q[i:i + 1], kc, vc, rag.dec_bt[i], lens[i], lens[i] - 1, H, G, dk, dv, scale, chunk, window,
-                          sink, out[i:i + 1], out_scale, sink_v, bias, gate[i:i + 1] if gate is not None else None, Gv)
+                          sink, out[i:i + 1], out_scale, sink_v, bias, gate[i:i + 1] if gate is not None else None, Gv, keep)
         if rag.n_pf:
             cu, ctx = rag.pf_cu.tolist(), rag.pf_ctx.tolist()
             for k in range(rag.n_pf):
@@ -465,7 +517,7 @@ def masked_attention(q: torch.Tensor, kc: torch.Tensor, vc: torch.Tensor, rag: R
                     r0 = nd + cu[k]
                     _attn_ref(q[r0:r0 + n], kc, vc, rag.pf_bt[k], ctx[k], ctx[k] - n, H, G, dk, dv, scale, chunk,
                               window, sink, out[r0:r0 + n], out_scale, sink_v, bias,
-                              gate[r0:r0 + n] if gate is not None else None, Gv)
+                              gate[r0:r0 + n] if gate is not None else None, Gv, keep)
         return out
     if q.dtype != kc.dtype or kc.dtype != vc.dtype or q.stride(1) != 1 or out.stride(1) != 1:
         raise TypeError("masked_attention: queries and pools share one dtype, rows are contiguous")
@@ -479,7 +531,7 @@ def masked_attention(q: torch.Tensor, kc: torch.Tensor, vc: torch.Tensor, rag: R
         bool(N.hybrid_kernels().mxh_attention_mfma_ok(dk, dv))
     if nd:
         vis = rag.dec_max_len
-        vis = min(vis, chunk) if chunk else min(vis, window) if window else vis
+        vis = min(vis, chunk) if chunk else min(vis, window + keep) if window else vis
         dec_mfma = mfma_ok and H // G <= 16  # a wave's 16 rows are the query heads of one key / value head
         parts, plen = 1, 0
         if workspace is not None:
@@ -495,12 +547,12 @@ def masked_attention(q: torch.Tensor, kc: torch.Tensor, vc: torch.Tensor, rag: R
                     rag.dec_bt.data_ptr(), rag.dec_bt.stride(0), rag.dec_lens.data_ptr(), nd, out.data_ptr(),
                     out.stride(0), _is16(out), H, G, dk, dv, float(scale), int(chunk), int(window), int(sink),
                     float(out_scale), parts, plen if parts > 1 else 0, N.ptr(ml), N.ptr(po), *extra, N.ptr(gate), ldg,
-                    Gv, int(p32), st)
+                    Gv, int(p32), int(keep), st)
         else:
             N.kcall("mxh_attention", q.data_ptr(), q.stride(0), _is16(q), kc.data_ptr(), vc.data_ptr(), bs,
                     rag.dec_bt.data_ptr(), rag.dec_bt.stride(0), None, rag.dec_lens.data_ptr(), nd, nd, 0,
                     out.data_ptr(), out.stride(0), _is16(out), *common, 0, parts, plen if parts > 1 else 0, N.ptr(ml),
-                    N.ptr(po), *extra, N.ptr(gate), ldg, Gv, st)
+                    N.ptr(po), *extra, N.ptr(gate), ldg, Gv, int(keep), st)
     if rag.n_pf:
         lens = rag.pf_q_host if len(rag.pf_q_host) == rag.n_pf and len(rag.pf_ctx_host) == rag.n_pf else None
 
@@ -508,7 +560,7 @@ def masked_attention(q: torch.Tensor, kc: torch.Tensor, vc: torch.Tensor, rag: R
             N.kcall("mxh_attention", q.data_ptr(), q.stride(0), _is16(q), kc.data_ptr(), vc.data_ptr(), bs,
                     rag.pf_bt.data_ptr(), rag.pf_bt.stride(0), rag.pf_cu.data_ptr(), rag.pf_ctx.data_ptr(), rag.n_pf,
                     n_rows, nd, out.data_ptr(), out.stride(0), _is16(out), *common, row_off, 1, 0, None, None, *extra,
-                    N.ptr(gate), ldg, Gv, st)
+                    N.ptr(gate), ldg, Gv, int(keep), st)
         mfma = mfma_ok
         big = MFMA_MIN_ROWS if mfma else GEMM_MIN_ROWS
         if lens is None or max(lens) < big or (not mfma and 0 < chunk < GEMM_MIN_ROWS):
@@ -526,10 +578,10 @@ def masked_attention(q: torch.Tensor, kc: torch.Tensor, vc: torch.Tensor, rag: R
                     N.kcall("mxh_attention_mfma", qk.data_ptr(), qk.stride(0), kc.data_ptr(), vc.data_ptr(), bs,
                             rag.pf_bt[k].data_ptr(), rag.pf_ctx_host[k] - n, n, ok.data_ptr(), ok.stride(0), _is16(out),
                             H, G, dk, dv, float(scale), int(chunk), int(window), int(sink), float(out_scale), *extra,
-                            N.ptr(gk), ldg, Gv, int(p32), st)
+                            N.ptr(gk), ldg, Gv, int(p32), int(keep), st)
                 else:
                     _attn_gemm_chunk(qk, kc, vc, rag.pf_bt[k], rag.pf_ctx_host[k] - n, n, H, G, dk, dv, scale, chunk,
-                                     window, sink, ok, out_scale, sink_v, bias, gk, Gv, p32)
+                                     window, sink, ok, out_scale, sink_v, bias, gk, Gv, p32, keep)
             elif n and run0 is None:
                 run0 = r
             r += n
@@ -779,22 +831,24 @@ def diff_group_norm(a: torch.Tensor, b: torch.Tensor, lam: float, eps: float, gr
 
 
 # ------------------------------------------------------------------------------------------------ feed-forward
-GLU_ACTS = {"silu": 0, "gelu_tanh": 1, "relu2": 2}
+GLU_ACTS = {"silu": 0, "gelu_tanh": 1, "relu2": 2, "clamped": 3}
 
 
 def glu(a: torch.Tensor, b: torch.Tensor | None, bias_a: torch.Tensor | None, bias_b: torch.Tensor | None,
         out: torch.Tensor, scale: torch.Tensor | None = None, group: int = 0, scale_sigmoid: bool = False,
-        act: str = "silu"):
+        act: str = "silu", limit: float = 0.0, alpha: float = 0.0):
     """out = act(a + bias_a) * (b + bias_b) [* factor] with act "silu" or "gelu_tanh" (0.5 z (1 + tanh(sqrt(2 / pi)
     (z + 0.044715 z^3)))); a, b fp32 [T, F] column slices, out fp32 or bf16 [T, F] (may be a column slice). `scale`
     fp32 [T, F / group] (column slice allowed) gives one factor per row and group of `group` columns, passed through a
     sigmoid first with `scale_sigmoid`. act "relu2" has no second operand (b = None) and the factor multiplies the
-    INPUT: out = relu(factor * (a + bias_a))^2, an expert that is fed its routing weight times the token."""
+    INPUT: out = relu(factor * (a + bias_a))^2, an expert that is fed its routing weight times the token.
+    act "clamped": out = g sigmoid(alpha g) (u + 1) [* factor] with g = min(a + bias_a, limit) and
+    u = clamp(b + bias_b, -limit, limit)."""
     T, Fn = a.shape
     if T == 0 or Fn == 0:
         return out
     if act not in GLU_ACTS or (b is None) != (act == "relu2"):
-        raise ValueError("glu: act is silu | gelu_tanh with two operands, or relu2 with one")
+        raise ValueError("glu: act is silu | gelu_tanh | clamped with two operands, or relu2 with one")
     if not a.is_cuda:
         x = a.float() + bias_a if bias_a is not None else a.float()
         s = None
@@ -805,7 +859,11 @@ def glu(a: torch.Tensor, b: torch.Tensor | None, bias_a: torch.Tensor | None, bi
             z = torch.relu(x * s if s is not None else x).pow(2)
         else:
             y = b.float() + bias_b if bias_b is not None else b.float()
-            z = (F.silu(x) if act == "silu" else F.gelu(x, approximate="tanh")) * y
+            if act == "clamped":
+                g = x.clamp(max=limit)
+                z = g * torch.sigmoid(alpha * g) * (y.clamp(-limit, limit) + 1.0)
+            else:
+                z = (F.silu(x) if act == "silu" else F.gelu(x, approximate="tanh")) * y
             if s is not None:
                 z = z * s
         out.copy_(z.to(out.dtype))
@@ -818,38 +876,48 @@ def glu(a: torch.Tensor, b: torch.Tensor | None, bias_a: torch.Tensor | None, bi
     N.kcall("mxh_glu", a.data_ptr(), a.stride(0), N.ptr(b), b.stride(0) if b is not None else 0, N.ptr(bias_a),
             N.ptr(bias_b), N.ptr(scale), scale.stride(0) if scale is not None else 0,
             group if scale is not None else Fn, int(scale_sigmoid), out.data_ptr(), out.stride(0), _is16(out), T, Fn,
-            GLU_ACTS[act], N.stream_ptr())
+            GLU_ACTS[act], float(limit), float(alpha), N.stream_ptr())
     return out
 
 
+ROUTE_MODES = {"softmax": 0, "sigmoid": 1, "scores": 2}
+
+
 def moe_route(logits: torch.Tensor, top: int, scale: float, weights: torch.Tensor, eps: float = 1e-20,
-              bias: torch.Tensor | None = None, mode: str = "softmax"):
+              bias: torch.Tensor | None = None, mode: str = "softmax", groups=None):
     """Router of a mixture of experts: s = softmax(logits + bias) over all E experts, the `top` largest are kept,
     divided by their sum (+ eps) and multiplied by `scale` (eps = 0, scale = 1: the softmax over the chosen logits
     alone). logits fp32 [T, E] (column slice allowed), bias fp32 [E]; weights fp32 [T, E] contiguous: the chosen
     experts' weights, 0 elsewhere. Ties go to the lower expert index. mode "sigmoid": the scores are
     sigmoid(logits + bias), the `top` largest are chosen and keep their scores as weights, times `scale`, not
-    renormalised."""
+    renormalised; mode "scores": the same with the softmax scores over all experts. `groups` = (count, keep): the experts
+    form `count` equal groups of neighbours and only those of the `keep` groups with the largest best scores can be
+    chosen (ties: the lower group)."""
     T, E = logits.shape
     if T == 0:
         return weights
     if not 0 < top <= E:
         raise ValueError("moe_route: 1 <= top <= experts")
-    if mode not in ("softmax", "sigmoid"):
-        raise ValueError("moe_route: softmax or sigmoid scores")
+    if mode not in ROUTE_MODES:
+        raise ValueError("moe_route: softmax, sigmoid or plain scores")
+    gc, gk = (int(groups[0]), int(groups[1])) if groups else (1, 1)
+    if gc < 1 or E % gc or not 1 <= gk <= gc or top > gk * (E // gc):
+        raise ValueError("moe_route: equal groups, and enough experts in the kept ones")
     if not logits.is_cuda:
         z = logits.float() + bias.float() if bias is not None else logits.float()
-        weights.zero_()
-        if mode == "sigmoid":
-            tv, ti = torch.topk(z, top, dim=-1)
-            weights.scatter_(1, ti, torch.sigmoid(tv) * scale)
-            return weights
-        tv, ti = torch.topk(torch.softmax(z, -1), top, dim=-1)
-        weights.scatter_(1, ti, tv / (tv.sum(-1, keepdim=True) + eps) * scale)
-        return weights
+        zs = z  # softmax and sigmoid order the experts as their logits do
+        if gc > 1:
+            best = z.reshape(T, gc, E // gc).max(-1).values
+            ok = torch.zeros_like(best, dtype=torch.bool).scatter_(1, torch.topk(best, gk, dim=-1).indices, True)
+            zs = z.masked_fill(~ok.repeat_interleave(E // gc, 1), float("-inf"))
+        ti = torch.topk(zs, top, dim=-1).indices
+        tv = (torch.sigmoid(z) if mode == "sigmoid" else torch.softmax(z, -1)).gather(1, ti)
+        if mode == "softmax":
+            tv = tv / (tv.sum(-1, keepdim=True) + eps)
+        return weights.zero_().scatter_(1, ti, tv * scale)
     _f32c(logits, "moe_route")
     if E > 1024:
         raise ValueError("moe_route: at most 1024 experts")
     N.kcall("mxh_moe_route", logits.data_ptr(), logits.stride(0), N.ptr(bias), T, E, top, float(scale), float(eps),
-            weights.data_ptr(), int(mode == "sigmoid"), N.stream_ptr())
+            weights.data_ptr(), ROUTE_MODES[mode], gc, gk, N.stream_ptr())
     return weights
