@@ -192,6 +192,10 @@ struct Sched {
                     o_pre.push_back(1);
                     continue;
                 }
+                // not admitted: matched blocks go back (they stay cached), or running sequences could not grow into them
+                free_blocks(sl);
+                f(F_NC, sl) = f(F_NCACHED, sl) = 0;
+                q.hashes.clear();
                 break;
             }
             waiting.pop_front();

@@ -181,6 +181,10 @@ class Scheduler:
                     s.finish_reason = "error:kv_cache_full"
                     out.preempted.append(s)
                     continue
+                # not admitted: matched blocks go back (they stay cached), or running sequences could not grow into them
+                self.free(s)
+                s.num_computed = s.num_cached = 0
+                s.block_hashes = []
                 break
             self.waiting.popleft()
             s.status = Status.RUNNING
