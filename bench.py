@@ -96,13 +96,13 @@ def parse():
                     help="comma list of sampling phases measured back to back on the same server: reference = "
                          "the reference's defaults (temperature 0.9, top_k 40, top_p 0.95; backend_config.go "
                          "SetDefaults) on the GPU sampler; greedy = argmax. The first phase is the headline")
-    ap.add_argument("--arch-bench", default="", choices=["", "vosotar", "vugotar", "girulorn", "keronex"],
+    ap.add_argument("--arch-bench", default="", choices=["", "vosotar", "vugotar", "girulorn", "keronex", "zomolix"],
                     help="instead of the headline serving benchmark: prefill and decode throughput of this model "
                          "family beside the Llama graph at equal layer sizes (random bf16 / f16 weights, one GPU)")
     ap.add_argument("--arch-sizes", default="1b,7b", help="--arch-bench: comma list of layer sizes (1b, 7b)")
     ap.add_argument("--arch-layers", type=int, default=4, help="--arch-bench: layers per model")
     ap.add_argument("--arch-models", default="", help="--arch-bench: comma list to restrict the models (vosotar, vugotar, girulorn, "
-                         "keronex, vugotar-moe, llama-f16)")
+                         "keronex, zomolix, vugotar-moe, llama-f16)")
     ap.add_argument("--arch-batches", default="1,32", help="--arch-bench: decode batch sizes")
     ap.add_argument("--arch-chunk", type=int, default=2048, help="--arch-bench vugotar: attention chunk size")
     return ap.parse_args()
@@ -283,6 +283,34 @@ def run_arch_bench(args) -> int:
                                 d_conv=4, m_heads=2 * s["hidden"] // 64, m_vdim=64, m_state=128, m_groups=1,
                                 m_norm_groups=1, m_conv=4, name=f"vugotar-{sz}", **moe)
             yield "vugotar-moe", lambda: VU.VugotarModel.load(uc, VU.synthetic_source(uc, 1), dev, torch.bfloat16)
+        elif args.arch_bench == "zomolix":
+            # two latent layers (512-wide latent, 64 rotated numbers) around a windowed attention layer and one that
+            # borrows its keys; attention heads as the Llama graph's (GQA 4:1, head size 128), a window of half the prompt
+            # with 16 kept tokens, scaled rotations; 8 experts in 4 groups of a quarter of the feed-forward width, two
+            # chosen, and a shared expert of half of it. Beside it the framework's two closest models: Vosotar (latent
+            # attention of the same rank in every layer, dense feed-forward of the full width) and Girulorn (attention
+            # with borrowed keys and sinks, gated linear attention, the same expert feed-forwards).
+            from localai_tfp_amd.models import girulorn as GI
+            from localai_tfp_amd.models import zomolix as ZO
+            kinds = ("latent_attention", "attention", "attention", "latent_attention")
+            moe = dict(experts=8, top=2, expert_ff=s["ff"] // 4, shared_ff=s["ff"] // 2)
+            kv = max(1, s["heads"] // 4)
+            zc = ZO.make_config(hidden=s["hidden"], vocab=V, pattern=tuple(kinds[i % 4] for i in range(nl)),
+                                kv_from={i: i - 1 for i in range(2, nl, 4)}, heads=s["heads"], kv_heads=kv, dim=128,
+                                vdim=128, window=P // 2, keep_first=16, rot_dims=64, rot_scaling=(4.0, 8192.0, 32.0, 1.0),
+                                l_heads=s["heads"], l_dim=128, l_rot=64, l_vdim=128, kv_rank=512,
+                                l_rot_scaling=(16.0, 4096.0, 32.0, 1.0), groups=(4, 2), limit=7.0, name=f"zomolix-{sz}",
+                                **moe)
+            yield "zomolix", lambda: ZO.ZomolixModel.load(zc, ZO.synthetic_source(zc, 1), dev, torch.bfloat16)
+            vc = VO.make_config(hidden=s["hidden"], vocab=V, n_layers=nl, heads=s["heads"], dim=128, vdim=128,
+                                kv_rank=512, q_rank=s["q_rank"], ff=s["ff"], name=f"vosotar-{sz}")
+            yield "vosotar", lambda: VO.VosotarModel.load(vc, VO.synthetic_source(vc, 1), dev, torch.bfloat16)
+            gc = GI.make_config(hidden=s["hidden"], vocab=V, pattern=tuple("gla" if i % 2 else "attention" for i in range(nl)),
+                                heads=s["heads"], kv_heads=kv, dim=128, vdim=128, bias_max=4096.0, bias_rows=64,
+                                temp_coef=0.25, temp_every=1024, kv_from={i: i - 2 for i in range(2, nl, 4)},
+                                g_heads=s["heads"] // 2, g_dim=128, g_vdim=128, tau=12.0, rank=32, name=f"girulorn-{sz}",
+                                **moe)
+            yield "girulorn", lambda: GI.GirulornModel.load(gc, GI.synthetic_source(gc, 1), dev, torch.bfloat16)
         elif args.arch_bench == "vugotar":
             # attention + delta-rule layers with a state-space layer every fourth, dense feed-forwards; attention
             # heads as the Llama graph's (GQA 4:1, head size 128), delta rule with half as many heads of 128 x 128
