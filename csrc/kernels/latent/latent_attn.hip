@@ -309,8 +309,10 @@ MX_DEV float group_sum16(float v) {
 // exchange, no extra barrier), each accumulates and writes one half of the output columns. Half the accumulators per
 // wave let two waves share a SIMD at the widest ranks, which is what hides the latencies between a tile's steps.
 // NVT: 16-column tiles of the value part (NVT * 16 >= R; all of the row unless the row has many key-only numbers).
+// The widest rows keep one wave per SIMD where two would spill or would not arise anyway (two-wave workgroups).
 template <int RV, int NVT, int NW, int RS>
-__global__ __launch_bounds__(NW * 64) __attribute__((amdgpu_waves_per_eu(RS == 2 ? 2 : 1)))
+__global__ __launch_bounds__(NW * 64)
+__attribute__((amdgpu_waves_per_eu(RS == 2 && !(RV > 12 && NW == 2) && RV <= 18 ? 2 : 1)))
 void latent_attn_mfma_kernel(AttnArgs a) {
     constexpr int RP = RV * 32, KT = 32, CSTR = RP * 2 + 16, PSTR = KT * 2 + 16, NTH = NW * 64;
     constexpr int BM = NW / RS * 16, NO = NVT / RS;  // rows per workgroup, output column tiles per wave
@@ -404,7 +406,9 @@ void latent_attn_mfma_kernel(AttnArgs a) {
     // current tile's products and stay in registers meanwhile (all of a tile when NTH * UB covers it); the rest
     // is loaded UB pieces at a time once the tile's turn has come.
     const int bs_shift = (a.bs & (a.bs - 1)) == 0 ? __builtin_ctz(a.bs) : -1;
-    constexpr int CPK = RP / 8, TOTAL = KT * CPK, UB = NW == 8 && RV > 16 ? 5 : (NW == 1 && RV > 8) || NW == 8 || (RS == 2 && RV > 12) ? 4 : 8;  // register room at the widest ranks
+    constexpr int CPK = RP / 8, TOTAL = KT * CPK, UB =  // register room at the widest ranks
+        RS == 2 && NW == 2 && RV > 12 ? RV / 2 : RS == 2 && RV > 16 ? (NW == 4 && RV > 18 ? 4 : 5)
+        : (NW == 1 && RV > 8) || NW == 8 || (RS == 2 && RV > 12) ? 4 : 8;
     u32x4 pre[UB];
     auto fetch = [&](int k0, int base, u32x4* v) {
 #pragma unroll
