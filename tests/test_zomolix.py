@@ -142,7 +142,7 @@ def test_clamped_unit_and_group_limited_router(dev):
     out = torch.empty(T, 33, device=dev)
     HY.glu(a.to(dev), b.to(dev), None, None, out, scale=rw.to(dev), group=11, act="clamped", limit=1.5, alpha=1.702)
     close(out, O.clamped_unit(a.double(), b.double(), 1.5) * rw.double().repeat_interleave(11, 1), 1e-5)
-    for E, top, groups in ((8, 4, (4, 3)), (8, 1, (8, 1)), (12, 4, (3, 1)), (6, 6, (2, 2)), (5, 2, None), (128, 6, (16, 3)),
+    for E, top, groups in ((8, 3, (4, 3)), (8, 1, (8, 1)), (12, 4, (3, 1)), (6, 6, (2, 2)), (5, 2, None), (128, 6, (16, 3)),
                            (320, 8, (20, 2)), (9, 3, (9, 5))):
         lg = torch.randn(T, E + 1, generator=g) * 2
         lg[0, 1:] += torch.arange(E).float() * 0.01  # (rows whose best experts crowd together)
@@ -299,7 +299,7 @@ def test_kept_tokens_need_a_window():
 
 @pytest.mark.parametrize("dev,dt", [("cpu", "float32"), pytest.param("cuda", "float32", marks=pytest.mark.gpu),
                                     pytest.param("cuda", "bfloat16", marks=pytest.mark.gpu)])
-@pytest.mark.parametrize("R,rot,H,d", [(40, 8, 3, 12), (21, 6, 2, 20), (96, 32, 4, 32), (512, 64, 16, 24), (512, 64, 20, 8),
+@pytest.mark.parametrize("R,rot,H,d", [(40, 8, 3, 12), (21, 6, 2, 20), (104, 24, 4, 40), (512, 64, 16, 24), (512, 64, 20, 8),
                                        (256, 64, 40, 16), (130, 2, 2, 6), (300, 40, 1, 16), (576, 64, 2, 8), (64, 0, 4, 16)])
 def test_latent_rows_with_a_rotated_part(dev, dt, R, rot, H, d):
     """Norm + rotation + append of (latent, rotated key part), the split of the queries, and attention over the rows with
@@ -478,13 +478,13 @@ def test_peaked_attention_far_keys_and_long_decode(dev, dt, tol):
 
 
 @pytest.mark.parametrize("dev,dt,tol", RUNS)
-@pytest.mark.parametrize("dim,vdim,heads,kv,rank,lrot", [(64, 128, 8, 2, 96, 32), (128, 64, 3, 1, 512, 64)])
+@pytest.mark.parametrize("dim,vdim,heads,kv,rank,lrot", [(64, 128, 8, 2, 80, 48), (128, 64, 3, 1, 512, 64)])
 def test_matrix_core_sizes_through_the_engine(dev, dt, tol, dim, vdim, heads, kv, rank, lrot):
     """Head sizes of 64 / 128 and latent rows of the matrix-core kernels: a prompt in portions that end inside 16-row
     tiles, decoded rows behind enough keys to be split into partitions."""
     kw = dict(hidden=128, vocab=211, pattern=("attention", "latent_attention", "attention"), kv_from={2: 0}, heads=heads,
               kv_heads=kv, dim=dim, vdim=vdim, scale=1.5 * dim ** -0.5, window=100, keep_first=6, rot_dims=dim // 2,
-              rot_scaling=(2.0, 128.0, 16.0, 1.0), l_heads=4, l_dim=32, l_rot=lrot, l_vdim=32, kv_rank=rank,
+              rot_scaling=(2.0, 128.0, 16.0, 1.0), l_heads=6, l_dim=32, l_rot=lrot, l_vdim=24, kv_rank=rank,
               experts=4, top=2, groups=(2, 1), expert_ff=64, shared_ff=64, emb_scale=2.0)
     cfg, tensors, model = build(dev, dt, seed=17, **kw)
     t = toks(330, cfg.vocab, 9)
@@ -632,7 +632,7 @@ def test_decode_graphs_equal_eager_steps_in_bf16():
     """The matrix-core decode kernels inside replayed graphs: many replays with the program's own work between them give
     the tokens of the eager engine (the same kernels, launched one by one)."""
     kw = dict(hidden=128, vocab=211, pattern=("attention", "latent_attention", "attention"), kv_from={2: 0}, heads=8,
-              kv_heads=2, dim=64, vdim=64, window=40, keep_first=4, l_heads=4, l_dim=32, l_rot=32, l_vdim=32, kv_rank=96,
+              kv_heads=2, dim=64, vdim=64, window=40, keep_first=4, l_heads=5, l_dim=24, l_rot=16, l_vdim=40, kv_rank=80,
               experts=4, top=2, groups=(2, 1), expert_ff=64, shared_ff=64)
     cfg, _, model = build("cuda", "bfloat16", seed=3, **kw)
     out = []
