@@ -6,12 +6,14 @@
 * `scale_add_norm`: x += (y + bias) * s with one factor per column (layer scale) and, in the same pass, the norm of the
   new residual that the next sublayer reads;
 * `rope_norm_append`: projection biases, rotary positions on neighbouring pairs (or half pairs) of the first `rot_dims`
-  numbers of each query / key head, by base^(-2i/d) or by given frequencies with a magnitude (scaled rotations), an optional unit-RMS norm of every head after the rotation (with optional per-channel weights), an optional
+  numbers of each query / key head, by base^(-2i/d) or by given frequencies with a magnitude (scaled rotations), an
+  optional unit-RMS norm of every head after the rotation (with optional per-channel weights), an optional
   position-dependent query temperature, and the append of keys and values to paged pools;
-* `masked_attention`: causal attention over the paged pools whose visible range starts at a chunk border
-  (`chunk`), `window` keys back (with the first `keep` tokens still visible), or at position 0, with an optional sink (one extra term exp(0), or exp(s_h) with a
-  learned s_h per head, in the softmax denominator that carries no value), an optional additive bias that depends on
-  the distance between query and key (`log_bucket_table`) and an optional sigmoid gate per token and head;
+* `masked_attention`: causal attention over the paged pools whose visible range starts at a chunk border (`chunk`),
+  `window` keys back (with the first `keep` tokens still visible), or at position 0, with an optional sink (one extra
+  term exp(0), or exp(s_h) with a learned s_h per head, in the softmax denominator that carries no value), an optional
+  additive bias that depends on the distance between query and key (`log_bucket_table`) and an optional sigmoid gate per
+  token and head;
 * `causal_conv`: a per-channel causal convolution over time (optional bias and SiLU) whose last taps-1 inputs are
   carried per sequence;
 * `unit_norm_heads`, `scan_coefs`, `channel_decay`, `state_scan`: the pieces of a linear recurrence
@@ -431,7 +433,8 @@ def _visible_blocks(p0: int, n: int, chunk: int, window: int, heads: int):
 def _attn_gemm_chunk(q, kc, vc, table, p0, n, H, G, dk, dv, scale, chunk, window, sink, out, out_scale, sink_v=None,
                      bias=None, gate=None, Gv=None, p32=False, keep=0):
     """A long prompt chunk (rows q [n, H*dk] at positions p0 ..) as library GEMMs: per block of rows, the visible keys
-    and values (with a window also the `keep` first tokens) are gathered head-major from the pages, scores = Q K^T (fp32), masked sink softmax, out = P V (fp32).
+    and values (with a window also the `keep` first tokens) are gathered head-major from the pages, scores = Q K^T
+    (fp32), masked sink softmax, out = P V (fp32).
     With `p32` and bf16 operands every softmax weight is written as two bf16 numbers (its rounding and the rest), side
     by side along K, and the values are stacked twice: the product sees the weights to 16 bits of mantissa."""
     from .dense import bmm_f32
@@ -472,7 +475,8 @@ def masked_attention(q: torch.Tensor, kc: torch.Tensor, vc: torch.Tensor, rag: R
     bf16's mantissa also in bf16 mode (the row kernels keep them in fp32 anyway; the matrix-core kernels and the GEMM
     route split each weight into two bf16 numbers, its rounding and the rounding of the rest). The row at position i
     sees j in [lo, i]: lo = (i // chunk) * chunk with `chunk`, max(0, i - window + 1) with `window`, else 0; with a
-    window the positions below `keep` stay visible as well, at their true distance. `sink` = True adds exp(0) to the softmax denominator, an fp32 tensor
+    window the positions below `keep` stay visible as well, at their true distance. `sink` = True adds
+    exp(0) to the softmax denominator, an fp32 tensor
     [H] adds exp(sink[h]). `bias` (fp32 [H, L], contiguous) adds bias[h, min(i - j, L - 1)] to the scaled score.
     `gate` (fp32 [T, H], may be a column slice) multiplies head h's output of row t by sigmoid(gate[t, h]). out
     [T, H*dv] (may be a column slice; fp32 or bf16) receives out_scale times the result. q, pools and out share fp32

@@ -302,13 +302,13 @@ def latent_attention(qa: torch.Tensor, cache: torch.Tensor, rag: Ragged, scale: 
                 parts = max(1, room)
                 part_len = -(-(-(-rag.dec_max_len // parts)) // 32) * 32
         ml, po = (workspace[0], workspace[1]) if parts > 1 else (None, None)
-        N.kcall("mxl_latent_attn", qa.data_ptr(), qa.stride(1), qa.stride(0), cache.data_ptr(), _is16(cache), bs, W, R, N.ptr(sink),
-                rag.dec_bt.data_ptr(), rag.dec_bt.stride(0), None, rag.dec_lens.data_ptr(), nd, nd, 0,
+        N.kcall("mxl_latent_attn", qa.data_ptr(), qa.stride(1), qa.stride(0), cache.data_ptr(), _is16(cache), bs, W, R,
+                N.ptr(sink), rag.dec_bt.data_ptr(), rag.dec_bt.stride(0), None, rag.dec_lens.data_ptr(), nd, nd, 0,
                 out.data_ptr(), out.stride(1), out.stride(0), float(scale), H, parts, part_len if parts > 1 else 0,
                 N.ptr(ml), N.ptr(po), impl, st)
     if rag.n_pf:
-        N.kcall("mxl_latent_attn", qa.data_ptr(), qa.stride(1), qa.stride(0), cache.data_ptr(), _is16(cache), bs, W, R, N.ptr(sink),
-                rag.pf_bt.data_ptr(), rag.pf_bt.stride(0), rag.pf_cu.data_ptr(), rag.pf_ctx.data_ptr(), rag.n_pf,
+        N.kcall("mxl_latent_attn", qa.data_ptr(), qa.stride(1), qa.stride(0), cache.data_ptr(), _is16(cache), bs, W, R,
+                N.ptr(sink), rag.pf_bt.data_ptr(), rag.pf_bt.stride(0), rag.pf_cu.data_ptr(), rag.pf_ctx.data_ptr(), rag.n_pf,
                 T - nd, nd, out.data_ptr(), out.stride(1), out.stride(0), float(scale), H, 1, 0, None, None, impl, st)
     return out
 
