@@ -4,8 +4,8 @@
 // The value pool may hold fewer heads than the key pool (gv of them, a divisor of G): key head g then reads value head
 // g % gv, several attention maps over the same values. Every kernel also takes an AttnExtra: a learned sink score per
 // head instead of 0, an additive bias looked up by the distance between query and key (table [H, distances], the last
-// entry serving every larger distance), a gate per row and head whose sigmoid multiplies the head's output, and a count
-// of first tokens (`keep`) that stay visible in front of a window.
+// entry serving every larger distance), a gate per row and head (or per row, head and value column) whose sigmoid multiplies the
+// output, a cap of the scores, and a count of first tokens (`keep`) that stay visible in front of a window.
 //
 // attn_rows_kernel: one wave per (query row, query head). Keys are taken 64 at a time, one per lane: the lane forms
 // its key's whole score against the query (held in LDS as fp32, pre-multiplied by the scale), the wave updates the
@@ -15,7 +15,7 @@
 // With parts > 1 (decode rows of long contexts) grid.z splits a row's visible keys into partitions whose
 // (max, sum, unnormalised output) go to a workspace; attn_merge_kernel combines them in a fixed order and adds the sink.
 //
-// bf16 pools with head sizes of 64 / 128 run on the matrix cores instead: attn_chunk_mfma_kernel for prompt chunks,
+// bf16 pools with head sizes of 64 / 128 (or 96 for both) run on the matrix cores instead: attn_chunk_mfma_kernel for prompt chunks,
 // attn_decode_mfma_kernel for single new tokens (both further down, with their fragment layouts).
 //
 // Other long prompt chunks take another route (ops/hybrid.py): kv_gather_kernel copies the chunk's visible keys and values
@@ -31,8 +31,10 @@ struct AttnExtra {
     const float* sink_v;  // [H] sink scores (null: 0 where a sink is asked for)
     const float* bias;    // [H, nb] bias by distance (null: none)
     int nb;
-    const float* gate;    // pre-sigmoid gate of row r and head h at gate[r * ldg + h] (null: none)
+    const float* gate;    // pre-sigmoid gate of row r and head h at gate[r * ldg + h * gw (+ value column)] (null: none)
     int ldg;
+    int gw;               // gates per head: 1, or one per value column
+    float softcap;        // > 0: scaled scores become softcap * tanh(score / softcap), before the bias and the mask
     int gv;               // value heads in the pool: key head g reads value head g % gv
     int keep;             // with a window: positions 0 .. keep - 1 stay visible whatever their distance
 };
@@ -50,8 +52,13 @@ MX_DEV float sink_score(const AttnExtra& ex, int h) { return ex.sink_v ? ex.sink
 MX_DEV float dist_bias(const AttnExtra& ex, int dist, int H, int h) {
     return ex.bias[(long)h * ex.nb + min(max(dist, 0), ex.nb - 1)];
 }
-MX_DEV float gate_factor(const AttnExtra& ex, long row, int h) {
-    return ex.gate ? 1.f / (1.f + expf(-ex.gate[row * ex.ldg + h])) : 1.f;
+MX_DEV float gate_factor(const AttnExtra& ex, long row, int h, int c) {
+    return ex.gate ? 1.f / (1.f + expf(-ex.gate[row * ex.ldg + (long)h * ex.gw + (ex.gw > 1 ? c : 0)])) : 1.f;
+}
+// Capped score times log2 e of a raw score s on the matrix-core routes: cap tanh(x) = cap - 2 cap / (exp(2 x) + 1) with
+// c2 = cap log2 e and k2 = 2 scale log2 e / cap. Errors are a few 1e-7 of the cap, far below the operands' rounding.
+MX_DEV float capped_log2(float s, float c2, float k2) {
+    return c2 - 2.f * c2 * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(s * k2) + 1.f);
 }
 
 template <bool B16>
@@ -192,6 +199,10 @@ __global__ __launch_bounds__(64) void attn_rows_kernel(const void* q, int ldq, c
         if (ok) {
             tok = (long)table[j / bs] * bs + (j % bs);
             dot_row<B16, REP>(kc, (tok * G + g) * dk, qs, dk, sc);
+            if (ex.softcap > 0.f) {
+#pragma unroll
+                for (int i = 0; i < REP; ++i) sc[i] = ex.softcap * tanhf(sc[i] / ex.softcap);
+            }
             if (ex.bias) {
 #pragma unroll
                 for (int i = 0; i < REP; ++i) sc[i] += dist_bias(ex, qpos - j, H, h0 + i);
@@ -259,14 +270,15 @@ __global__ __launch_bounds__(64) void attn_rows_kernel(const void* q, int ldq, c
             }
             continue;
         }
-        const float inv = out_scale / l[i] * gate_factor(ex, row_base + r, h);
+        const float inv = out_scale / l[i];
         const long orow = (long)(row_base + r) * ldo + (long)h * dv;
 #pragma unroll
         for (int u = 0; u < DVU; ++u) {
             const int c = lane + u * 64;
             if (c < dv) {
-                if constexpr (O16) ((bf16_t*)out)[orow + c] = f32_to_bf16(acc[i][u] * inv);
-                else ((float*)out)[orow + c] = acc[i][u] * inv;
+                const float v = acc[i][u] * (inv * gate_factor(ex, row_base + r, h, c));
+                if constexpr (O16) ((bf16_t*)out)[orow + c] = f32_to_bf16(v);
+                else ((float*)out)[orow + c] = v;
             }
         }
     }
@@ -417,6 +429,19 @@ __global__ __launch_bounds__(256) void attn_chunk_mfma_kernel(const bf16_t* __re
                 sacc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qf[ks], kf, sacc[t], 0, 0, 0);
             }
         }
+        // ---- scale (and cap): sacc is in base 2 from here on ----
+        if (ex.softcap > 0.f) {
+            const float c2 = ex.softcap * LOG2E_, k2 = 2.f * qs / ex.softcap;
+#pragma unroll
+            for (int t = 0; t < 4; ++t)
+#pragma unroll
+                for (int i = 0; i < 4; ++i) sacc[t][i] = capped_log2(sacc[t][i], c2, k2);
+        } else {
+#pragma unroll
+            for (int t = 0; t < 4; ++t)
+#pragma unroll
+                for (int i = 0; i < 4; ++i) sacc[t][i] *= qs;
+        }
         // ---- bias by distance: row 4g + i against key 16t + col lies d0 + i - 16t keys back. When every distance
         // of the wave's 16 rows against the tile's 64 keys lies inside the table (a wave-uniform test) the 16 entries
         // are read at constant offsets from one address; the diagonal tile and tiles beyond the table clamp ----
@@ -429,19 +454,14 @@ __global__ __launch_bounds__(256) void attn_chunk_mfma_kernel(const bf16_t* __re
 #pragma unroll
                 for (int t = 0; t < 4; ++t)
 #pragma unroll
-                    for (int i = 0; i < 4; ++i) sacc[t][i] = sacc[t][i] * qs + pp[i - 16 * t] * LOG2E_;
+                    for (int i = 0; i < 4; ++i) sacc[t][i] += pp[i - 16 * t] * LOG2E_;
             } else {
 #pragma unroll
                 for (int t = 0; t < 4; ++t)
 #pragma unroll
                     for (int i = 0; i < 4; ++i)
-                        sacc[t][i] = sacc[t][i] * qs + bp[min(max(d0 + i - 16 * t, 0), ex.nb - 1)] * LOG2E_;
+                        sacc[t][i] += bp[min(max(d0 + i - 16 * t, 0), ex.nb - 1)] * LOG2E_;
             }
-        } else {
-#pragma unroll
-            for (int t = 0; t < 4; ++t)
-#pragma unroll
-                for (int i = 0; i < 4; ++i) sacc[t][i] *= qs;
         }
         // ---- mask + online softmax in base 2 (rows 4g + i, keys 16t + col) ----
         float alpha[4];
@@ -504,12 +524,13 @@ __global__ __launch_bounds__(256) void attn_chunk_mfma_kernel(const bf16_t* __re
     for (int i = 0; i < 4; ++i) {
         const int qi = row_q0 + 4 * g + i;
         if (qi >= n) continue;
-        const float inv = lrow[i] > 0.f ? out_scale / lrow[i] * gate_factor(ex, qi, hq) : 0.f;
+        const float inv = lrow[i] > 0.f ? out_scale / lrow[i] : 0.f;
 #pragma unroll
         for (int nt = 0; nt < DV / 16; ++nt) {
             const size_t o = (size_t)qi * ldo + (size_t)hq * DV + 16 * nt + col;
-            if constexpr (O16) ((bf16_t*)out)[o] = f32_to_bf16(oacc[nt][i] * inv);
-            else ((float*)out)[o] = oacc[nt][i] * inv;
+            const float v = oacc[nt][i] * (inv * gate_factor(ex, qi, hq, 16 * nt + col));
+            if constexpr (O16) ((bf16_t*)out)[o] = f32_to_bf16(v);
+            else ((float*)out)[o] = v;
         }
     }
 }
@@ -612,6 +633,19 @@ __global__ __launch_bounds__(64) void attn_decode_mfma_kernel(const bf16_t* __re
                                                                   0, 0, 0);
         }
         if (kt0 + KT < v_end) load_tile(kt0 + KT);
+        // scale (and cap): sacc is in base 2 from here on
+        if (ex.softcap > 0.f) {
+            const float c2 = ex.softcap * LOG2E_, k2 = 2.f * qs / ex.softcap;
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+#pragma unroll
+                for (int t = 0; t < KT / 16; ++t) sacc[t][i] = capped_log2(sacc[t][i], c2, k2);
+        } else {
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+#pragma unroll
+                for (int t = 0; t < KT / 16; ++t) sacc[t][i] *= qs;
+        }
         // bias by distance: every row (query head) of the tile is at the same position, key 16t + col lies
         // d0 - 16t keys back (a tile that begins behind the kept tokens); each head has its own table row
         if (ex.bias && kt0 < kr.kn) {  // kept tokens and the window's first keys in one tile: distances one by one
@@ -619,7 +653,7 @@ __global__ __launch_bounds__(64) void attn_decode_mfma_kernel(const bf16_t* __re
             for (int t = 0; t < KT / 16; ++t) {
                 const int d = min(max(qpos - kr.pos(min(kt0 + 16 * t + col, v_end - 1)), 0), ex.nb - 1);
 #pragma unroll
-                for (int i = 0; i < 4; ++i) sacc[t][i] = sacc[t][i] * qs + ex.bias[(size_t)hrow[i] * ex.nb + d] * LOG2E_;
+                for (int i = 0; i < 4; ++i) sacc[t][i] += ex.bias[(size_t)hrow[i] * ex.nb + d] * LOG2E_;
             }
         } else if (ex.bias) {
             const int d0 = qpos - kr.gap - kt0 - col;
@@ -630,14 +664,9 @@ __global__ __launch_bounds__(64) void attn_decode_mfma_kernel(const bf16_t* __re
 #pragma unroll
                 for (int t = 0; t < KT / 16; ++t) {
                     const int d = inside ? d0 - 16 * t : min(max(d0 - 16 * t, 0), ex.nb - 1);
-                    sacc[t][i] = sacc[t][i] * qs + bp[d] * LOG2E_;
+                    sacc[t][i] += bp[d] * LOG2E_;
                 }
             }
-        } else {
-#pragma unroll
-            for (int i = 0; i < 4; ++i)
-#pragma unroll
-                for (int t = 0; t < KT / 16; ++t) sacc[t][i] *= qs;
         }
         float alpha[4];
 #pragma unroll
@@ -704,12 +733,13 @@ __global__ __launch_bounds__(64) void attn_decode_mfma_kernel(const bf16_t* __re
             for (int nt = 0; nt < DV / 16; ++nt) part_o[pr * DV + 16 * nt + col] = oacc[nt][i];
             continue;
         }
-        const float inv = lrow[i] > 0.f ? out_scale / lrow[i] * gate_factor(ex, s, h) : 0.f;
+        const float inv = lrow[i] > 0.f ? out_scale / lrow[i] : 0.f;
 #pragma unroll
         for (int nt = 0; nt < DV / 16; ++nt) {
             const size_t o = (size_t)s * ldo + (size_t)h * DV + 16 * nt + col;
-            if constexpr (O16) ((bf16_t*)out)[o] = f32_to_bf16(oacc[nt][i] * inv);
-            else ((float*)out)[o] = oacc[nt][i] * inv;
+            const float v = oacc[nt][i] * (inv * gate_factor(ex, s, h, 16 * nt + col));
+            if constexpr (O16) ((bf16_t*)out)[o] = f32_to_bf16(v);
+            else ((float*)out)[o] = v;
         }
     }
 }
@@ -735,7 +765,7 @@ __global__ __launch_bounds__(64) void attn_merge_kernel(const float* part_ml, co
     if (sink) M = fmaxf(M, s0);
     const float w = lz > 0.f ? expf(mz - M) : 0.f;
     const float L = wave_sum(lz * w) + (sink ? expf(s0 - M) : 0.f);
-    const float inv = out_scale / L * gate_factor(ex, row_base + r, h);
+    const float inv = out_scale / L;
     const long orow = (long)(row_base + r) * ldo + (long)h * dv;
 #pragma unroll
     for (int u = 0; u < DVU; ++u) {
@@ -751,8 +781,9 @@ __global__ __launch_bounds__(64) void attn_merge_kernel(const float* part_ml, co
                 for (int e = 0; e < 8; ++e) a += x[e] * __shfl(w, min(z0 + e, 63), 64) * (z0 + e < parts ? 1.f : 0.f);
             }
             if (c < dv) {
-                if constexpr (O16) ((bf16_t*)out)[orow + c] = f32_to_bf16(a * inv);
-                else ((float*)out)[orow + c] = a * inv;
+                const float v = a * (inv * gate_factor(ex, row_base + r, h, c));
+                if constexpr (O16) ((bf16_t*)out)[orow + c] = f32_to_bf16(v);
+                else ((float*)out)[orow + c] = v;
             }
         }
     }
@@ -778,11 +809,12 @@ __global__ __launch_bounds__(64) void kv_gather_kernel(const E* kc, const E* vc,
 // grid (n, H): dst[i * d_si + h * d_sh + e] = scale * src[i * s_si + h * s_sh + e], e < d
 template <bool S16, bool D16>
 __global__ __launch_bounds__(64) void head_transpose_kernel(const void* src, long s_si, long s_sh, void* dst, long d_si,
-                                                            long d_sh, int d, float scale, const float* gate, int ldg) {
+                                                            long d_sh, int d, float scale, const float* gate, int ldg,
+                                                            int gw) {
     const long so = blockIdx.x * s_si + blockIdx.y * s_sh, dof = blockIdx.x * d_si + blockIdx.y * d_sh;
-    if (gate) scale /= 1.f + expf(-gate[(long)blockIdx.x * ldg + blockIdx.y]);  // sigmoid gate of (row, head)
+    const float* gr = gate ? gate + (long)blockIdx.x * ldg + (long)blockIdx.y * gw : nullptr;  // sigmoid gates of (row, head)
     for (int e = threadIdx.x; e < d; e += 64) {
-        const float v = ld1<S16>(src, so + e) * scale;
+        const float v = ld1<S16>(src, so + e) * (gr ? scale / (1.f + expf(-gr[gw > 1 ? e : 0])) : scale);
         if constexpr (D16) ((bf16_t*)dst)[dof + e] = f32_to_bf16(v);
         else ((float*)dst)[dof + e] = v;
     }
@@ -796,7 +828,7 @@ template <bool P16>
 __global__ __launch_bounds__(256) void masked_softmax_kernel(const float* sc, void* pw, int n, int nk, int p0, int key0,
                                                              float scale, int chunk, int window, int sink,
                                                              const float* sink_v, const float* bias, int nb, int H,
-                                                             int two, int kn, int keep) {
+                                                             int two, int kn, int keep, float softcap) {
     __shared__ float red[4];
     const long row = blockIdx.x;
     const int i = (int)(row % n), h = (int)(row / n);
@@ -811,7 +843,9 @@ __global__ __launch_bounds__(256) void masked_softmax_kernel(const float* sc, vo
     auto score = [&](int j) {
         const int p = j < kn ? j : j + gap;
         if (p < lo && p >= keep) return -INFINITY;
-        return s[j] * scale + (bias ? bias[(long)h * nb + min(pos - p, nb - 1)] : 0.f);
+        float x = s[j] * scale;
+        if (softcap > 0.f) x = softcap * tanhf(x / softcap);
+        return x + (bias ? bias[(long)h * nb + min(pos - p, nb - 1)] : 0.f);
     };
     float m = sink ? s0 : -INFINITY;
     for (int j = a + threadIdx.x; j <= b; j += 256) m = fmaxf(m, score(j));
@@ -846,10 +880,11 @@ extern "C" int mxh_attention(const void* q, int ldq, int q16, const void* kc, co
                              void* out, int ldo, int o16, int H, int G, int dk, int dv, float scale, int chunk,
                              int window, int sink, float out_scale, int row_off, int parts, int part_len,
                              float* part_ml, float* part_o, const float* sink_v, const float* bias, int nb,
-                             const float* gate, int ldg, int gv, int keep, hipStream_t st) {
+                             const float* gate, int ldg, int gv, int keep, int gw, float softcap, hipStream_t st) {
     if (n_rows <= 0 || n_seqs <= 0) return 0;
-    MXH_CHECK((!bias || nb > 0) && (!gate || ldg >= H) && (!sink_v || sink) && gv > 0 && G % gv == 0 && keep >= 0);
-    const AttnExtra ex = {sink_v, bias, nb, gate, ldg, gv, keep};
+    MXH_CHECK((!bias || nb > 0) && (!gate || ldg >= H * gw) && (!sink_v || sink) && gv > 0 && G % gv == 0 && keep >= 0);
+    MXH_CHECK((gw == 1 || gw == dv) && softcap >= 0.f);
+    const AttnExtra ex = {sink_v, bias, nb, gate, ldg, gw, softcap, gv, keep};
     MXH_CHECK(q && kc && vc && bt && ctx && out && bs > 0 && bt_stride > 0);
     MXH_CHECK(H > 0 && G > 0 && H % G == 0 && dk > 0 && dv > 0 && dv <= 64 * DVU_MAX && dk <= 4096);
     MXH_CHECK(ldq >= H * dk && ldo >= H * dv && chunk >= 0 && window >= 0 && H <= 65535 && row_off >= 0);
@@ -898,12 +933,12 @@ extern "C" int mxh_kv_gather(const void* kc, const void* vc, int is16, int bs, c
 }
 
 extern "C" int mxh_head_transpose(const void* src, int s16, long s_si, long s_sh, void* dst, int d16, long d_si,
-                                  long d_sh, int n, int H, int d, float scale, const float* gate, int ldg,
+                                  long d_sh, int n, int H, int d, float scale, const float* gate, int ldg, int gw,
                                   hipStream_t st) {
     if (n <= 0) return 0;
-    MXH_CHECK(src && dst && H > 0 && H <= 65535 && d > 0 && (!gate || ldg >= H));
+    MXH_CHECK(src && dst && H > 0 && H <= 65535 && d > 0 && (!gate || ((gw == 1 || gw == d) && ldg >= H * gw)));
     const dim3 grid(n, H);
-#define GO(S, D) head_transpose_kernel<S, D><<<grid, 64, 0, st>>>(src, s_si, s_sh, dst, d_si, d_sh, d, scale, gate, ldg)
+#define GO(S, D) head_transpose_kernel<S, D><<<grid, 64, 0, st>>>(src, s_si, s_sh, dst, d_si, d_sh, d, scale, gate, ldg, gw)
     if (s16 && d16) GO(true, true);
     else if (s16) GO(true, false);
     else if (d16) GO(false, true);
@@ -914,32 +949,36 @@ extern "C" int mxh_head_transpose(const void* src, int s16, long s_si, long s_sh
 
 extern "C" int mxh_masked_softmax(const float* sc, void* pw, int p16, long rows, int n, int nk, int p0, int key0,
                                   float scale, int chunk, int window, int sink, const float* sink_v,
-                                  const float* bias, int nb, int H, int two, int kn, int keep, hipStream_t st) {
+                                  const float* bias, int nb, int H, int two, int kn, int keep, float softcap,
+                                  hipStream_t st) {
     if (rows <= 0) return 0;
     MXH_CHECK((!two || p16) && kn >= 0 && kn <= key0 && kn <= nk && keep >= 0);
     MXH_CHECK(sc && pw && n > 0 && nk > 0 && rows % n == 0 && rows < (1L << 31) && key0 >= 0 && p0 >= key0);
     MXH_CHECK((!bias || nb > 0) && (!(bias || sink_v) || rows == (long)H * n));
     if (p16)
         masked_softmax_kernel<true><<<(unsigned)rows, 256, 0, st>>>(sc, pw, n, nk, p0, key0, scale, chunk, window, sink,
-                                                                    sink_v, bias, nb, H, two, kn, keep);
+                                                                    sink_v, bias, nb, H, two, kn, keep, softcap);
     else
         masked_softmax_kernel<false><<<(unsigned)rows, 256, 0, st>>>(sc, pw, n, nk, p0, key0, scale, chunk, window, sink,
-                                                                     sink_v, bias, nb, H, 0, kn, keep);
+                                                                     sink_v, bias, nb, H, 0, kn, keep, softcap);
     return (int)hipGetLastError();
 }
 
 // A prompt chunk of n rows of one sequence (q and out point at its first row) at positions p0 .., bf16 pools.
 // Returns hipErrorInvalidValue for head sizes without an instantiation: the caller asks mxh_attention_mfma_ok first.
-extern "C" int mxh_attention_mfma_ok(int dk, int dv) { return (dk == 64 || dk == 128) && (dv == 64 || dv == 128); }
+extern "C" int mxh_attention_mfma_ok(int dk, int dv) {
+    return ((dk == 64 || dk == 128) && (dv == 64 || dv == 128)) || (dk == 96 && dv == 96);
+}
 
 extern "C" int mxh_attention_mfma(const void* q, int ldq, const void* kc, const void* vc, int bs, const int* table,
                                   int p0, int n, void* out, int ldo, int o16, int H, int G, int dk, int dv,
                                   float scale, int chunk, int window, int sink, float out_scale, const float* sink_v,
                                   const float* bias, int nb, const float* gate, int ldg, int gv, int p2,
-                                  int keep, hipStream_t st) {
+                                  int keep, int gw, float softcap, hipStream_t st) {
     if (n <= 0) return 0;
-    MXH_CHECK((!bias || nb > 0) && (!gate || ldg >= H) && (!sink_v || sink) && gv > 0 && G % gv == 0 && keep >= 0);
-    const AttnExtra ex = {sink_v, bias, nb, gate, ldg, gv, keep};
+    MXH_CHECK((!bias || nb > 0) && (!gate || ldg >= H * gw) && (!sink_v || sink) && gv > 0 && G % gv == 0 && keep >= 0);
+    MXH_CHECK((gw == 1 || gw == dv) && softcap >= 0.f);
+    const AttnExtra ex = {sink_v, bias, nb, gate, ldg, gw, softcap, gv, keep};
     MXH_CHECK(q && kc && vc && table && out && bs > 0 && p0 >= 0 && H > 0 && G > 0 && H % G == 0);
     MXH_CHECK(mxh_attention_mfma_ok(dk, dv) && ldq >= H * dk && ldq % 8 == 0 && ldo >= H * dv && chunk >= 0 && window >= 0);
     const int rep = H / G;
@@ -961,6 +1000,7 @@ extern "C" int mxh_attention_mfma(const void* q, int ldq, const void* kc, const 
     if (dk == 64 && dv == 64) GO(64, 64);
     else if (dk == 64 && dv == 128) GO(64, 128);
     else if (dk == 128 && dv == 64) GO(128, 64);
+    else if (dk == 96) GO(96, 96);
     else GO(128, 128);
 #undef GO
 #undef GO3
@@ -974,10 +1014,11 @@ extern "C" int mxh_attention_decode_mfma(const void* q, int ldq, const void* kc,
                                          int G, int dk, int dv, float scale, int chunk, int window, int sink,
                                          float out_scale, int parts, int part_len, float* part_ml, float* part_o,
                                          const float* sink_v, const float* bias, int nb, const float* gate, int ldg,
-                                         int gv, int p2, int keep, hipStream_t st) {
+                                         int gv, int p2, int keep, int gw, float softcap, hipStream_t st) {
     if (n_seqs <= 0) return 0;
-    MXH_CHECK((!bias || nb > 0) && (!gate || ldg >= H) && (!sink_v || sink) && gv > 0 && G % gv == 0 && keep >= 0);
-    const AttnExtra ex = {sink_v, bias, nb, gate, ldg, gv, keep};
+    MXH_CHECK((!bias || nb > 0) && (!gate || ldg >= H * gw) && (!sink_v || sink) && gv > 0 && G % gv == 0 && keep >= 0);
+    MXH_CHECK((gw == 1 || gw == dv) && softcap >= 0.f);
+    const AttnExtra ex = {sink_v, bias, nb, gate, ldg, gw, softcap, gv, keep};
     MXH_CHECK(q && kc && vc && bt && ctx && out && bs > 0 && bt_stride > 0 && H > 0 && G > 0 && H % G == 0);
     MXH_CHECK(H / G <= 16 && G <= 65535 && mxh_attention_mfma_ok(dk, dv) && ldq >= H * dk && ldq % 8 == 0 && ldo >= H * dv);
     MXH_CHECK(parts >= 1 && parts <= 64 && (parts == 1 || (part_len > 0 && part_ml && part_o)) && chunk >= 0 && window >= 0);
@@ -996,6 +1037,7 @@ extern "C" int mxh_attention_decode_mfma(const void* q, int ldq, const void* kc,
     if (dk == 64 && dv == 64) GO(64, 64);
     else if (dk == 64 && dv == 128) GO(64, 128);
     else if (dk == 128 && dv == 64) GO(128, 64);
+    else if (dk == 96) GO(96, 96);
     else GO(128, 128);
 #undef GO
 #undef GO3

@@ -153,13 +153,14 @@ __global__ __launch_bounds__(1024) void norm_add_kernel(const float* y, int ldy,
     }
 }
 
-// x[t] += (y[t] + b) * s (b, s per column, either may be null: 0 / 1); with w also the norm that follows,
+// x[t] += (y[t] + b) * s * mult (b, s per column, either may be null: 0 / 1); with w also the norm that follows,
 // h = x[t] / rms(x[t]) * (offset + w), as fp32 and / or bf16. One block per row (256 or 1024 threads); rows of up to
 // nt * RK numbers keep the new x in registers between the two.
 template <int RK>
 __global__ __launch_bounds__(1024) void scale_add_norm_kernel(const float* y, int ldy, const float* b, const float* s,
                                                               float* x, int ldx, const float* w, float offset, float eps,
-                                                              float* o32, int ld32, bf16_t* o16, int ld16, int C) {
+                                                              float* o32, int ld32, bf16_t* o16, int ld16, int C,
+                                                              float mult) {
     __shared__ float red[16];
     const int i = blockIdx.x, nt = blockDim.x;
     const float* yr = y + (long)i * ldy;
@@ -175,7 +176,7 @@ __global__ __launch_bounds__(1024) void scale_add_norm_kernel(const float* y, in
             yk[k] = yr[c];
             xk[k] = xr[c];
             bk[k] = b ? b[c] : 0.f;
-            sk[k] = s ? s[c] : 1.f;
+            sk[k] = s ? s[c] * mult : mult;
             wk[k] = w ? w[c] : 0.f;
         }
 #pragma unroll
@@ -189,7 +190,7 @@ __global__ __launch_bounds__(1024) void scale_add_norm_kernel(const float* y, in
         }
     } else {
         for (int c = threadIdx.x; c < C; c += nt) {
-            const float v = xr[c] + (yr[c] + (b ? b[c] : 0.f)) * (s ? s[c] : 1.f);
+            const float v = xr[c] + (yr[c] + (b ? b[c] : 0.f)) * (s ? s[c] * mult : mult);
             xr[c] = v;
             ss += v * v;
         }
@@ -414,6 +415,7 @@ __global__ __launch_bounds__(NT) void channel_decay_kernel(const float* z, int l
 // the smallest GC that holds the group
 // sigm: the gate's activation is a sigmoid instead of a SiLU. proj [R, C]: the gate row holds R numbers and column
 // c's pre-activation is sum_r gate[t, r] proj[r, c], summed in fp32 in a fixed order (a low-rank gate's second half).
+// den, den_min (one number per row and group, ldd apart): the group is first divided by max(|den|, den_min) + den_eps.
 MX_DEV float gate_act(float x, int sigm) { return sigm ? sigmoid_acc(x) : silu_acc(x); }
 MX_DEV float gate_pre(const float* gr, const float* proj, int R, int C, int c, const float* zr) {
     if (!proj) return gr[c];
@@ -424,11 +426,14 @@ MX_DEV float gate_pre(const float* gr, const float* proj, int R, int C, int c, c
 template <bool B16, int GC>
 __global__ void gated_group_norm_kernel(const float* y, int ldy, const float* gate, int ldg, const float* w, int wlen,
                                         float eps, int group, int gate_first, float out_scale, void* out, int ldo,
-                                        int sigm, const float* proj, int R, int C) {
+                                        int sigm, const float* proj, int R, int C, const float* den,
+                                        const float* den_min, int ldd, float den_eps) {
     __shared__ float red[16];
     extern __shared__ float zr[];  // the token's R inputs of the gate projection
     const int t = blockIdx.x, c0 = blockIdx.y * group;
     const float* yr = y + (long)t * ldy + c0;
+    const long di = (long)t * ldd + blockIdx.y;
+    const float inv = den ? 1.f / (fmaxf(fabsf(den[di]), den_min[di]) + den_eps) : 1.f;
     const float* gr = gate + (long)t * ldg + (proj ? 0 : c0);
     const int nt = blockDim.x;
     if (proj) {  // the general form below, with the projected gate
@@ -436,7 +441,7 @@ __global__ void gated_group_norm_kernel(const float* y, int ldy, const float* ga
         __syncthreads();
         float ss = 0.f;
         for (int e = threadIdx.x; e < group; e += nt) {
-            float v = yr[e];
+            float v = yr[e] * inv;
             if (gate_first) v *= gate_act(gate_pre(gr, proj, R, C, c0 + e, zr), sigm);
             ss += v * v;
         }
@@ -444,7 +449,7 @@ __global__ void gated_group_norm_kernel(const float* y, int ldy, const float* ga
         const float sc = out_scale / sqrtf(ss / (float)group + eps);
         for (int e = threadIdx.x; e < group; e += nt) {
             const float g = gate_act(gate_pre(gr, proj, R, C, c0 + e, zr), sigm);
-            float v = yr[e];
+            float v = yr[e] * inv;
             if (gate_first) v *= g;
             v = v * sc * w[(c0 + e) % wlen];
             if (!gate_first) v *= g;
@@ -465,6 +470,7 @@ __global__ void gated_group_norm_kernel(const float* y, int ldy, const float* ga
         for (int k = 0; k < GC; ++k) {
             const int e = threadIdx.x + k * nt;
             gs[k] = gate_act(gs[k], sigm);
+            z[k] *= inv;
             z[k] = e < group ? (gate_first ? z[k] * gs[k] : z[k]) : 0.f;
             ss += z[k] * z[k];
         }
@@ -483,7 +489,7 @@ __global__ void gated_group_norm_kernel(const float* y, int ldy, const float* ga
     }
     float ss = 0.f;
     for (int e = threadIdx.x; e < group; e += nt) {
-        float v = yr[e];
+        float v = yr[e] * inv;
         if (gate_first) v *= gate_act(gr[e], sigm);
         ss += v * v;
     }
@@ -491,7 +497,7 @@ __global__ void gated_group_norm_kernel(const float* y, int ldy, const float* ga
     const float sc = out_scale / sqrtf(ss / (float)group + eps);
     for (int e = threadIdx.x; e < group; e += nt) {
         const float g = gate_act(gr[e], sigm);
-        float v = yr[e];
+        float v = yr[e] * inv;
         if (gate_first) v *= g;
         v = v * sc * w[(c0 + e) % wlen];
         if (!gate_first) v *= g;
@@ -502,6 +508,7 @@ __global__ void gated_group_norm_kernel(const float* y, int ldy, const float* ga
 // grid (T, ceil(F / NT))
 // act 0: silu(x) * y * factor; 1: gelu_tanh(x) * y * factor; 2 (no second operand): relu(factor * x)^2;
 // 3: g sigmoid(alpha g) (u + 1) * factor with g = min(x, limit), u = clamp(y, -limit, limit)
+// 4 (no second operand): gelu(x) * factor, the exact form with erf
 MX_DEV float gelu_tanh_acc(float x) {
     return 0.5f * x * (1.f + tanhf(0.7978845608028654f * (x + 0.044715f * x * x * x)));
 }
@@ -525,6 +532,10 @@ __global__ __launch_bounds__(NT) void glu_kernel(const float* a, int lda, const 
     if (act == 2) {
         const float r = fmaxf(fac * x, 0.f);
         st_elem<B16>(out, (long)t * ldo + f, r * r);
+        return;
+    }
+    if (act == 4) {
+        st_elem<B16>(out, (long)t * ldo + f, 0.5f * x * (1.f + erff(x * 0.7071067811865476f)) * fac);
         return;
     }
     const float y = b[(long)t * ldb + f] + (bb ? bb[f] : 0.f);
@@ -668,10 +679,10 @@ extern "C" int mxh_norm_add(const float* y, int ldy, const float* w, float offse
 
 extern "C" int mxh_scale_add_norm(const float* y, int ldy, const float* b, const float* s, float* x, int ldx,
                                   const float* w, float offset, float eps, float* o32, int ld32, bf16_t* o16, int ld16,
-                                  int T, int C, hipStream_t st) {
+                                  int T, int C, float mult, hipStream_t st) {
     if (T <= 0) return 0;
     MXH_CHECK(y && x && C > 0 && ldy >= C && ldx >= C && (!w || o32 || o16) && (!o32 || ld32 >= C) && (!o16 || ld16 >= C));
-#define GO(K_, nt_) scale_add_norm_kernel<K_><<<T, nt_, 0, st>>>(y, ldy, b, s, x, ldx, w, offset, eps, o32, ld32, o16, ld16, C)
+#define GO(K_, nt_) scale_add_norm_kernel<K_><<<T, nt_, 0, st>>>(y, ldy, b, s, x, ldx, w, offset, eps, o32, ld32, o16, ld16, C, mult)
     if (C <= 1024) GO(4, 256);
     else if (C <= 4096) GO(4, 1024);
     else GO(8, 1024);
@@ -750,15 +761,17 @@ extern "C" int mxh_channel_decay(const float* z, int ldz, const float* bias, flo
 
 extern "C" int mxh_gated_group_norm(const float* y, int ldy, const float* gate, int ldg, const float* w, int wlen,
                                     float eps, int group, int gate_first, float out_scale, void* out, int ldo,
-                                    int o16, int T, int C, int sigm, const float* proj, int R, hipStream_t st) {
+                                    int o16, int T, int C, int sigm, const float* proj, int R, const float* den,
+                                    const float* den_min, int ldd, float den_eps, hipStream_t st) {
     if (T <= 0) return 0;
     MXH_CHECK(y && gate && w && out && C > 0 && group > 0 && C % group == 0 && wlen > 0 && C % wlen == 0);
+    MXH_CHECK((!den || (den_min && ldd >= C / group)) && den_eps >= 0.f);
     MXH_CHECK(ldy >= C && ldo >= C && (proj ? (R > 0 && R <= 8192 && ldg >= R) : ldg >= C) && C / group <= 65535);
     const dim3 grid(T, C / group);
     const size_t dyn = proj ? R * sizeof(float) : 0;
 #define GO(B, G_, nt_)                                                                                              \
     gated_group_norm_kernel<B, G_><<<grid, nt_, dyn, st>>>(y, ldy, gate, ldg, w, wlen, eps, group, gate_first, out_scale, \
-                                                           out, ldo, sigm, proj, R, C)
+                                                           out, ldo, sigm, proj, R, C, den, den_min, ldd, den_eps)
 #define PICK(B)                              \
     do {                                     \
         if (group <= 256) GO(B, 4, 64);      \
@@ -777,8 +790,8 @@ extern "C" int mxh_glu(const float* a, int lda, const float* b, int ldb, const f
                        const float* scale, int lds, int group, int scale_sigmoid, void* out, int ldo, int o16, int T,
                        int F, int act, float limit, float alpha, hipStream_t st) {
     if (T <= 0 || F <= 0) return 0;
-    MXH_CHECK(a && out && lda >= F && ldo >= F && group > 0 && F <= 65535 * NT && act >= 0 && act <= 3);
-    MXH_CHECK(act == 2 ? !b : (b && ldb >= F));  // the squared ReLU has one operand
+    MXH_CHECK(a && out && lda >= F && ldo >= F && group > 0 && F <= 65535 * NT && act >= 0 && act <= 4);
+    MXH_CHECK(act == 2 || act == 4 ? !b : (b && ldb >= F));  // the squared ReLU and the plain gelu have one operand
     MXH_CHECK(!scale || (F % group == 0 && lds >= F / group));
     const dim3 grid(T, (F + NT - 1) / NT);
     if (o16)

@@ -16,6 +16,8 @@
 // missing write strength means 1, one given as pre-activations (coef_sigmoid, row stride ldc) passes a sigmoid when
 // staged; q_t is multiplied by q_scale when staged. A decay row stride of 0 (ldd) is one constant per head for every
 // token (retention).
+// nout: the state has one more column per head (P + 1 of them) whose value is 1 at every token, so it holds
+// n <- a_t n + c_t k_t; its product n^T q_t goes to nout [rows, H] (the normaliser of a matrix memory).
 #include "../mx_common.h"
 
 namespace {
@@ -43,7 +45,8 @@ __global__ __launch_bounds__(256) void state_scan_kernel(const float* k, int ldk
                                                          const float* coef, int ldc, int coef_sigmoid,
                                                          const float* skip, float* state, const int* seq_state,
                                                          const int* positions, int n_dec, const int* pf_cu, float* out,
-                                                         int ldo, int H, int G, int N, int P, float q_scale) {
+                                                         int ldo, int H, int G, int N, int P, float q_scale,
+                                                         float* nout) {
     static_assert(LPC == 4 || LPC == 16, "a column's lanes are a quad or a DPP row");
     constexpr int NT = 256;
     constexpr int NP = NPL * LPC;  // padded N
@@ -70,12 +73,13 @@ __global__ __launch_bounds__(256) void state_scan_kernel(const float* k, int ldk
     if (n <= 0) return;
     const int slot = seq_state[s];
     const bool fresh = positions[row0] == 0 || slot < 0;
-    const bool live = col < P;
+    const int PT = P + (nout ? 1 : 0);  // state columns of a head
+    const bool live = col < PT;
     const int g = h / (H / G);
     // addresses are clamped so that every load below is unconditional (all in flight together); what a lane must not
     // use is replaced by zero afterwards
-    const int colc = min(col, P - 1);
-    float* sp = state + (((long)(slot < 0 ? 0 : slot) * H + h) * P + colc) * N;
+    const int colc = min(col, PT - 1);
+    float* sp = state + (((long)(slot < 0 ? 0 : slot) * H + h) * PT + colc) * N;
     const bool whole = N == NP && (N & 3) == 0;  // no padding: a lane's run is NPL aligned floats
     float S[NPL];
     if (whole) {
@@ -161,7 +165,7 @@ __global__ __launch_bounds__(256) void state_scan_kernel(const float* k, int ldk
         for (int tt = 0; tt < nt; ++tt) {
             const int row = row0 + c * TB + tt;
             const float a = ac[b][tt][0], cf = ac[b][tt][1];
-            const float vv = live ? vs[b][tt][cl] : 0.f;
+            const float vv = col < P ? vs[b][tt][cl] : live ? 1.f : 0.f;
             const float* kb = &kq[b][tt][0][part * NPL];
             const float* qb = &kq[b][tt][1][part * NPL];
             float u;
@@ -195,7 +199,10 @@ __global__ __launch_bounds__(256) void state_scan_kernel(const float* k, int ldk
                 o1 += S[j + 1] * qb[j + 1];
             }
             const float o = lanes_sum<LPC>(o0 + o1);
-            if (live && part == 0) out[(long)row * ldo + (long)h * P + col] = o + sk * vv;
+            if (part == 0) {
+                if (col < P) out[(long)row * ldo + (long)h * P + col] = o + sk * vv;
+                else if (live) nout[(long)row * H + h] = o;
+            }
         }
         // the other buffer was last read while chunk c - 1 was worked on, before the barrier that ended that round
         if (c + 1 < nchunks) publish(b ^ 1);
@@ -214,6 +221,72 @@ __global__ __launch_bounds__(256) void state_scan_kernel(const float* k, int ldk
     }
 }
 
+// Scales of an exponentially gated matrix memory (ops/hybrid.py mlstm_gates). Per sequence and head, over the step's rows:
+//     i = cap tanh((zi + bi) / cap),  f = log sigmoid(cap tanh((zf + bf) / cap)),  m_t = max(f_t + m_(t-1), i_t)
+//     decay_t = exp(f_t + m_(t-1) - m_t),  coef_t = exp(i_t - m_t),  floor_t = exp(-m_t)
+// The running maximum is a scan of the maps m -> max(m + A, B), which compose to maps of the same form: a block takes
+// blockDim.x tokens at a time (a wave-wide prefix, the waves' totals through LDS), and every token reads its
+// predecessor's m as that one computed it, so stored states and scales always refer to the same number. m starts at 0
+// and is carried in peak[slot][h]. grid (H, sequences)
+__global__ __launch_bounds__(256) void mlstm_gates_kernel(const float* zi, const float* zf, int ldz, const float* bi,
+                                                          const float* bf, float cap, float* peak, const int* seq_state,
+                                                          const int* positions, int n_dec, const int* pf_cu,
+                                                          float* decay, float* coef, float* floor_, int H) {
+    __shared__ float ms[257];  // m of the token before the round's first, then of its tokens
+    __shared__ float ta[4], tb[4];  // a wave's 64 maps composed
+    const int h = blockIdx.x, s = blockIdx.y, nt = blockDim.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    int row0, n;
+    if (s < n_dec) {
+        row0 = s;
+        n = 1;
+    } else {
+        const int k = s - n_dec;
+        row0 = n_dec + pf_cu[k];
+        n = pf_cu[k + 1] - pf_cu[k];
+    }
+    if (n <= 0) return;
+    const int slot = seq_state[s];
+    const bool fresh = positions[row0] == 0 || slot < 0;
+    float m0 = fresh ? 0.f : peak[(long)slot * H + h];
+    const float b0 = bi ? bi[h] : 0.f, b1 = bf ? bf[h] : 0.f;
+    for (int base = 0; base < n; base += nt) {
+        const bool ok = base + tid < n;
+        const long row = row0 + min(base + tid, n - 1);
+        const float x = -cap * tanhf((zf[row * ldz + h] + b1) / cap);
+        const float gi = cap * tanhf((zi[row * ldz + h] + b0) / cap);
+        const float gf = -(x > 30.f ? x : log1pf(expf(x)));
+        float A = ok ? gf : 0.f, B = ok ? gi : -INFINITY;  // past the end: the identity
+#pragma unroll
+        for (int o = 1; o < 64; o <<= 1) {
+            const float Ap = __shfl_up(A, o, 64), Bp = __shfl_up(B, o, 64);
+            if (lane >= o) {
+                B = fmaxf(Bp + A, B);
+                A += Ap;
+            }
+        }
+        if (lane == 63) {
+            ta[wave] = A;
+            tb[wave] = B;
+        }
+        if (tid == 0) ms[0] = m0;
+        __syncthreads();
+        float m = m0;
+        for (int w = 0; w < wave; ++w) m = fmaxf(m + ta[w], tb[w]);
+        m = fmaxf(m + A, B);
+        ms[tid + 1] = m;
+        __syncthreads();
+        if (ok) {
+            const long o = row * H + h;
+            decay[o] = expf(gf + ms[tid] - m);
+            coef[o] = expf(gi - m);
+            floor_[o] = expf(-m);
+        }
+        m0 = ms[min(nt, n - base)];
+        __syncthreads();  // (the next round writes ms and the totals)
+    }
+    if (slot >= 0 && tid == 0) peak[(long)slot * H + h] = m0;
+}
+
 }  // namespace
 
 #define MXH_CHECK(cond) \
@@ -223,7 +296,7 @@ extern "C" int mxh_state_scan(const float* k, int ldk, const float* q, int ldq, 
                               const float* decay, int decay_rows, const float* coef, int ldc, int coef_sigmoid,
                               const float* skip, float* state, const int* seq_state, const int* positions, int n_dec,
                               const int* pf_cu, int n_pf, float* out, int ldo, int H, int G, int N, int P, int delta,
-                              int channel, float q_scale, hipStream_t st) {
+                              int channel, float q_scale, float* nout, hipStream_t st) {
     const int n_seqs = n_dec + n_pf;
     if (n_seqs <= 0) return 0;
     MXH_CHECK(k && q && v && decay && state && seq_state && positions && out && (n_pf == 0 || pf_cu));
@@ -234,11 +307,11 @@ extern "C" int mxh_state_scan(const float* k, int ldk, const float* q, int ldq, 
     const int lpc = N <= 32 ? 4 : 16;
     const int threads = 256;
     const int cols = threads / lpc;
-    const dim3 grid((P + cols - 1) / cols, H, n_seqs);
+    const dim3 grid((P + (nout ? 1 : 0) + cols - 1) / cols, H, n_seqs);
 #define GO2(NPL, LPC, D_, C_)                                                                                      \
     state_scan_kernel<NPL, LPC, D_, C_><<<grid, threads, 0, st>>>(k, ldk, q, ldq, v, ldv, decay, ldd, coef, ldc,      \
                                                                   coef_sigmoid, skip, state, seq_state, positions,    \
-                                                                  n_dec, pf_cu, out, ldo, H, G, N, P, q_scale)
+                                                                  n_dec, pf_cu, out, ldo, H, G, N, P, q_scale, nout)
 #define GO(NPL, LPC)                              \
     do {                                          \
         if (delta && channel) GO2(NPL, LPC, true, true); \
@@ -253,5 +326,17 @@ extern "C" int mxh_state_scan(const float* k, int ldk, const float* q, int ldq, 
     else GO(16, 16);
 #undef GO
 #undef GO2
+    return (int)hipGetLastError();
+}
+
+extern "C" int mxh_mlstm_gates(const float* zi, const float* zf, int ldz, const float* bi, const float* bf, float cap,
+                               float* peak, const int* seq_state, const int* positions, int n_dec, const int* pf_cu,
+                               int n_pf, float* decay, float* coef, float* floor_, int H, hipStream_t st) {
+    const int n_seqs = n_dec + n_pf;
+    if (n_seqs <= 0) return 0;
+    MXH_CHECK(zi && zf && peak && seq_state && positions && decay && coef && floor_ && (n_pf == 0 || pf_cu));
+    MXH_CHECK(H > 0 && ldz >= H && cap > 0.f && n_seqs <= 65535);
+    mlstm_gates_kernel<<<dim3(H, n_seqs), n_pf ? 256 : 64, 0, st>>>(zi, zf, ldz, bi, bf, cap, peak, seq_state, positions,
+                                                                    n_dec, pf_cu, decay, coef, floor_, H);
     return (int)hipGetLastError();
 }

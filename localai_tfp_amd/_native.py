@@ -151,8 +151,14 @@ HYBRID_SIGS = {
     "mxh_offset_norm": [P, I, P, P, F, F, P, I, P, I, I, I, P],
     # y, ldy, w, offset, eps, x, ldx, out16, ld16, T, C, stream
     "mxh_norm_add": [P, I, P, F, F, P, I, P, I, I, I, P],
-    # y, ldy, bias, scale, x, ldx, norm_w, offset, eps, out32, ld32, out16, ld16, T, C, stream
-    "mxh_scale_add_norm": [P, I, P, P, P, I, P, F, F, P, I, P, I, I, I, P],
+    # y, ldy, bias, scale, x, ldx, norm_w, offset, eps, out32, ld32, out16, ld16, T, C, factor, stream
+    "mxh_scale_add_norm": [P, I, P, P, P, I, P, F, F, P, I, P, I, I, I, F, P],
+    # q, ldq, k, ldk, v, ldv, positions, slots, H, G, dk, dv, rot_dims, half, freqs, mag, q_weight, k_weight, eps, conv_w,
+    # taps, tails, seq_state, n_dec, pf_cu, n_pf, q_out, ldqo, q16, kc, vc, c16, T, stream
+    "mxh_row_rope_append": [P, I, P, I, P, I, P, P, I, I, I, I, I, I, P, F, P, P, F, P, I, P, P, I, P, I, P, I, I, P, P, I,
+                            I, P],
+    # zi, zf, ldz, bias_i, bias_f, cap, peak, seq_state, positions, n_dec, pf_cu, n_pf, decay, coef, floor, H, stream
+    "mxh_mlstm_gates": [P, P, I, P, P, F, P, P, P, I, P, I, P, P, P, I, P],
     # q, k, v, ldq, ldk, ldv, positions, H, G, dk, dv, rot_dims, base, norm, eps, q_out, ldqo, q16, kc, vc, c16, slots,
     # q_weight, k_weight, temp_coef, temp_every, T, stream
     # ..., temp_every, half, value heads, freqs, mag, q_bias, k_bias, v_bias, T, stream
@@ -161,25 +167,26 @@ HYBRID_SIGS = {
     # q, ldq, q16, kc, vc, bs, bt, bt_stride, cu_q, ctx, n_seqs, n_rows, row_base, out, ldo, o16, H, G, dk, dv, scale,
     # chunk, window, sink, out_scale, row_off, parts, part_len, part_ml, part_o, sink_v, bias, bias_rows, gate, ldg,
     # stream
-    # (value heads and kept first tokens before the stream)
+    # (value heads, kept first tokens, gates per head and score cap before the stream)
     "mxh_attention": [P, I, I, P, P, I, P, I, P, P, I, I, I, P, I, I, I, I, I, I, F, I, I, I, F, I, I, I, P, P, P, P, I,
-                      P, I, I, I, P],
+                      P, I, I, I, I, F, P],
     # q, ldq, kc, vc, bs, table, p0, n, out, ldo, o16, H, G, dk, dv, scale, chunk, window, sink, out_scale, sink_v,
     # bias, bias_rows, gate, ldg, stream
-    # (value heads, the two-part weights flag and the kept first tokens before the stream)
-    "mxh_attention_mfma": [P, I, P, P, I, P, I, I, P, I, I, I, I, I, I, F, I, I, I, F, P, P, I, P, I, I, I, I, P],
+    # (value heads, the two-part weights flag, kept first tokens, gates per head and score cap before the stream)
+    "mxh_attention_mfma": [P, I, P, P, I, P, I, I, P, I, I, I, I, I, I, F, I, I, I, F, P, P, I, P, I, I, I, I, I,
+                           F, P],
     "mxh_attention_mfma_ok": [I, I],
     # q, ldq, kc, vc, bs, bt, bt_stride, ctx, n_seqs, out, ldo, o16, H, G, dk, dv, scale, chunk, window, sink, out_scale,
     # parts, part_len, part_ml, part_o, sink_v, bias, bias_rows, gate, ldg, stream
     "mxh_attention_decode_mfma": [P, I, P, P, I, P, I, P, I, P, I, I, I, I, I, I, F, I, I, I, F, I, I, P, P, P, P, I, P,
-                                  I, I, I, I, P],
+                                  I, I, I, I, I, F, P],
     # kc, vc, is16, bs, table, lo, n, G, dk, dv, kh, vh, value heads, kept first tokens, stream
     "mxh_kv_gather": [P, P, I, I, P, I, I, I, I, I, P, P, I, I, P],
-    # src, s16, s_stride_i, s_stride_h, dst, d16, d_stride_i, d_stride_h, n, H, d, scale, gate, ldg, stream
-    "mxh_head_transpose": [P, I, L, L, P, I, L, L, I, I, I, F, P, I, P],
+    # src, s16, s_stride_i, s_stride_h, dst, d16, d_stride_i, d_stride_h, n, H, d, scale, gate, ldg, gates per head, stream
+    "mxh_head_transpose": [P, I, L, L, P, I, L, L, I, I, I, F, P, I, I, P],
     # scores, weights, w16, rows, n, nk, p0, key0, scale, chunk, window, sink, sink_v, bias, bias_rows, H, two,
-    # columns of kept first tokens, kept first tokens, stream
-    "mxh_masked_softmax": [P, P, I, L, I, I, I, I, F, I, I, I, P, P, I, I, I, I, I, P],
+    # columns of kept first tokens, kept first tokens, score cap, stream
+    "mxh_masked_softmax": [P, P, I, L, I, I, I, I, F, I, I, I, P, P, I, I, I, I, I, F, P],
     # x, ldx, w, bias, taps, silu, tails, state, positions, n_dec, pf_cu, n_pf, out, ldo, T, C, stream
     "mxh_causal_conv": [P, I, P, P, I, I, P, P, P, I, P, I, P, I, I, I, P],
     # x, ldx, heads, dim, eps, scale, split, scale2, T, stream
@@ -189,10 +196,11 @@ HYBRID_SIGS = {
     # z, ldz, bias, 1 / tau, out, T, C, proj, R, stream
     "mxh_channel_decay": [P, I, P, F, P, I, I, P, I, P, I, P],
     # k, ldk, q, ldq, v, ldv, decay, coef, skip, state, seq_state, positions, n_dec, pf_cu, n_pf, out, ldo, H, G, N, P,
-    # delta, channel, q_scale, stream
-    "mxh_state_scan": [P, I, P, I, P, I, P, I, P, I, I, P, P, P, P, I, P, I, P, I, I, I, I, I, I, I, F, P],
-    # y, ldy, gate, ldg, w, wlen, eps, group, gate_first, out_scale, out, ldo, o16, T, C, sigmoid gate, proj, R, stream
-    "mxh_gated_group_norm": [P, I, P, I, P, I, F, I, I, F, P, I, I, I, I, I, P, I, P],
+    # delta, channel, q_scale, normaliser out, stream
+    "mxh_state_scan": [P, I, P, I, P, I, P, I, P, I, I, P, P, P, P, I, P, I, P, I, I, I, I, I, I, I, F, P, P],
+    # y, ldy, gate, ldg, w, wlen, eps, group, gate_first, out_scale, out, ldo, o16, T, C, sigmoid gate, proj, R, den, den_min,
+    # ldd, den_eps, stream
+    "mxh_gated_group_norm": [P, I, P, I, P, I, F, I, I, F, P, I, I, I, I, I, P, I, P, P, I, F, P],
     # a, lda, b, ldb, bias_a, bias_b, scale, lds, group, scale_sigmoid, out, ldo, o16, T, F, act, limit, alpha,
     # stream
     "mxh_glu": [P, I, P, I, P, P, P, I, I, I, P, I, I, I, I, I, F, F, P],

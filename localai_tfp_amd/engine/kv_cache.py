@@ -217,10 +217,11 @@ class HybridCache:
       head (ops/latent.py: a latent, with a rotated key part beside it), addressed the same way; None otherwise;
     * `state[i]`: fp32 [state_slots, heads, P, N] recurrent state (N numbers for each of a head's P value columns),
       None for runs without a recurrence;
-    * `tails[i]`: fp32 [state_slots, taps - 1, channels] last inputs of the run's causal convolution, or None.
+    * `tails[i]`: fp32 [state_slots, taps - 1, channels] last inputs of the run's causal convolution, or None;
+    * `peak[i]`: fp32 [state_slots, heads] running maximum of the run's exponential gates, or None.
 
     `spec` lists per run a dict with the optional keys "kv": (key row, value row), "lat": row, "state": (heads, P, N),
-    "tails": (taps - 1, channels). State slots are handed out per live sequence by `SlotPool`. With `seq_tokens` the
+    "tails": (taps - 1, channels), "peak": heads. State slots are handed out per live sequence by `SlotPool`. With `seq_tokens` the
     cache also carries `last_token` int32 [state_slots]: the newest token of each live sequence, for embeddings that
     look at the token before."""
 
@@ -231,7 +232,7 @@ class HybridCache:
         S = max(1, state_slots)
         f32 = dict(dtype=torch.float32, device=device)
         self.last_token = torch.zeros(S, dtype=torch.int32, device=device) if seq_tokens else None
-        self.kv, self.lat, self.state, self.tails = [], [], [], []
+        self.kv, self.lat, self.state, self.tails, self.peak = [], [], [], [], []
         for e in spec:
             row = e.get("lat")
             self.lat.append(None if row is None else
@@ -242,6 +243,8 @@ class HybridCache:
                             torch.zeros((num_blocks, block_size, int(kv[1])), dtype=dtype, device=device)))
             self.state.append(None if st is None else torch.zeros((S, *[int(x) for x in st]), **f32))
             self.tails.append(None if tl is None else torch.zeros((S, max(1, int(tl[0])), int(tl[1])), **f32))
+            pk = e.get("peak")
+            self.peak.append(None if pk is None else torch.zeros((S, int(pk)), **f32))
 
     def layer(self, i: int):
         return self.kv[i], self.state[i], self.tails[i]
@@ -252,7 +255,7 @@ class HybridCache:
         return [sum(e.get("kv") or ()) + int(e.get("lat") or 0) for e in spec if e.get("kv") or e.get("lat")]
 
     def state_bytes_per_seq(self) -> int:
-        return int(sum(t[0].numel() * 4 for t in self.state + self.tails if t is not None))
+        return int(sum(t[0].numel() * 4 for t in self.state + self.tails + self.peak if t is not None))
 
 
 class SlotPool:

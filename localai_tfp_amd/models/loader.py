@@ -153,18 +153,19 @@ def _state_families():
     `architecture`: name -> (module, model class name, config maker for `synthetic:<key>`)."""
     from . import girulorn as GI
     from . import keronex as KE
+    from . import tebodra as TE
     from . import vosotar as VO
     from . import vugotar as VU
     from . import zomolix as ZO
     return {"vosotar": (VO, VO.VosotarModel, VO.is_vosotar_dir), "vugotar": (VU, VU.VugotarModel, VU.is_vugotar_dir),
             "girulorn": (GI, GI.GirulornModel, GI.is_girulorn_dir), "keronex": (KE, KE.KeronexModel, KE.is_keronex_dir),
-            "zomolix": (ZO, ZO.ZomolixModel, ZO.is_zomolix_dir)}
+            "zomolix": (ZO, ZO.ZomolixModel, ZO.is_zomolix_dir), "tebodra": (TE, TE.TebodraModel, TE.is_tebodra_dir)}
 
 
 def _load_latent(model: str, device, tp_size: int, ov: dict):
     """Latent-attention decoders (models/vosotar.py, models/zomolix.py) and hybrid attention / recurrent decoders
-    (models/vugotar.py, models/girulorn.py, models/keronex.py): a directory whose config.json names the architecture, or
-    `synthetic:<family>-*` random weights. `overrides["dtype"]`: torch.bfloat16 (default on GPU) | torch.float32. None
+    (models/vugotar.py, models/girulorn.py, models/keronex.py, models/tebodra.py): a directory whose config.json names the
+    architecture, or `synthetic:<family>-*` random weights. `overrides["dtype"]`: torch.bfloat16 (default on GPU) | torch.float32. None
     for everything else."""
     from ..tokenizer import ByteTokenizer
     fam = None

@@ -3,17 +3,19 @@
 * `embed_rows`, `offset_rmsnorm`, `norm_add`: an fp32 residual from a 16-bit table; an RMS norm whose weight is
   stored around an offset (x / rms * (offset + w)); the same norm applied to a sublayer's OUTPUT and added to the
   residual (x += y / rms(y) * (offset + w)), with the 16-bit copy of the new residual the next GEMM reads;
-* `scale_add_norm`: x += (y + bias) * s with one factor per column (layer scale) and, in the same pass, the norm of the
-  new residual that the next sublayer reads;
+* `scale_add_norm`: x += (y + bias) * s with one factor per column (layer scale) and / or one factor for all and, in the
+  same pass, the norm of the new residual that the next sublayer reads;
 * `rope_norm_append`: projection biases, rotary positions on neighbouring pairs (or half pairs) of the first `rot_dims`
   numbers of each query / key head, by base^(-2i/d) or by given frequencies with a magnitude (scaled rotations), an
   optional unit-RMS norm of every head after the rotation (with optional per-channel weights), an optional
   position-dependent query temperature, and the append of keys and values to paged pools;
+* `row_rope_append`: the same step for layers whose queries and keys pass a short causal convolution over time, or an RMS
+  norm over the whole projection, before the rotation; also for values that are the keys before the rotation;
 * `masked_attention`: causal attention over the paged pools whose visible range starts at a chunk border (`chunk`),
   `window` keys back (with the first `keep` tokens still visible), or at position 0, with an optional sink (one extra
   term exp(0), or exp(s_h) with a learned s_h per head, in the softmax denominator that carries no value), an optional
-  additive bias that depends on the distance between query and key (`log_bucket_table`) and an optional sigmoid gate per
-  token and head;
+  additive bias that depends on the distance between query and key (`log_bucket_table`), an optional cap of the scores
+  (cap tanh(s / cap)) and an optional sigmoid gate per token and head, or per token, head and value column;
 * `causal_conv`: a per-channel causal convolution over time (optional bias and SiLU) whose last taps-1 inputs are
   carried per sequence;
 * `unit_norm_heads`, `scan_coefs`, `channel_decay`, `state_scan`: the pieces of a linear recurrence
@@ -21,8 +23,11 @@
   `delta` the written value is u = c (v - S^T k) after the decay (gated delta rule), otherwise u = c v with an
   optional skip D v on the output (state-space duality form); the decay a is one number per head or, for gated
   linear attention, one per key channel (S <- diag(a) S + k v^T, a = sigmoid(z)^(1/tau));
+* `mlstm_gates`: decays, write strengths and normaliser bounds of an exponentially gated matrix memory, whose running
+  maximum is carried per sequence; `state_scan` then keeps the normaliser as one more column of the state and
+  `gated_group_norm` divides by it;
 * `gated_group_norm`: unit-RMS norm over groups of columns, a weight, and a SiLU gate before or after the norm;
-* `glu`: silu(a + bias) * (b + bias), or other gated units (tanh gelu, squared ReLU, a clamped sigmoid unit), with an
+* `glu`: silu(a + bias) * (b + bias), or other units (tanh gelu, squared ReLU, a clamped sigmoid unit, plain gelu), with an
   optional per-row, per-column-group factor (routing weights of experts
   evaluated side by side, or the sigmoid gate of a shared expert);
 * `moe_route`: softmax over experts (optional logit bias), the `top` largest, renormalised and scaled, as a dense
@@ -120,9 +125,9 @@ def norm_add(y: torch.Tensor, w: torch.Tensor, eps: float, x: torch.Tensor, out1
 
 def scale_add_norm(y: torch.Tensor, bias: torch.Tensor | None, scale: torch.Tensor | None, x: torch.Tensor,
                    norm_w: torch.Tensor | None = None, eps: float = 0.0, out32: torch.Tensor | None = None,
-                   out16: torch.Tensor | None = None, offset: float = 0.0):
-    """x += (y + bias) * scale on fp32 rows [T, C] (bias, scale fp32 [C]; None: 0 and 1): a sublayer's output enters the
-    residual through a layer scale. With `norm_w` the same pass writes the norm the next sublayer reads,
+                   out16: torch.Tensor | None = None, offset: float = 0.0, mult: float = 1.0):
+    """x += (y + bias) * scale * mult on fp32 rows [T, C] (bias, scale fp32 [C]; None: 0 and 1): a sublayer's output enters
+    the residual through a layer scale or one factor. With `norm_w` the same pass writes the norm the next sublayer reads,
     x / sqrt(mean(x^2) + eps) * (offset + norm_w) of the new x, as fp32 (`out32`) and / or bf16 (`out16`)."""
     T, C = y.shape
     if T == 0:
@@ -131,7 +136,7 @@ def scale_add_norm(y: torch.Tensor, bias: torch.Tensor | None, scale: torch.Tens
         raise ValueError("scale_add_norm: a norm needs an output")
     if not y.is_cuda:
         z = y if bias is None else y + bias
-        x.add_(z if scale is None else z * scale)
+        x.add_((z if scale is None else z * scale) * mult)
         if norm_w is not None:
             offset_rmsnorm(x, norm_w, eps, out32, out16, offset=offset)
         return x
@@ -142,7 +147,7 @@ def scale_add_norm(y: torch.Tensor, bias: torch.Tensor | None, scale: torch.Tens
             raise TypeError("scale_add_norm: fp32 vectors of one number per column")
     N.kcall("mxh_scale_add_norm", y.data_ptr(), y.stride(0), N.ptr(bias), N.ptr(scale), x.data_ptr(), x.stride(0),
             N.ptr(norm_w), float(offset), float(eps), N.ptr(out32), out32.stride(0) if out32 is not None else 0,
-            N.ptr(out16), out16.stride(0) if out16 is not None else 0, T, C, N.stream_ptr())
+            N.ptr(out16), out16.stride(0) if out16 is not None else 0, T, C, float(mult), N.stream_ptr())
     return x
 
 
@@ -321,6 +326,73 @@ def rope_norm_append(q_in: torch.Tensor, k_in: torch.Tensor, v_in: torch.Tensor,
             float(mag), N.ptr(q_bias), N.ptr(k_bias), N.ptr(v_bias), T, N.stream_ptr())
 
 
+def row_rope_append(q_in: torch.Tensor, k_in: torch.Tensor | None, v_in: torch.Tensor | None, rag: Ragged, H: int, G: int,
+                    dk: int, dv: int, freqs: torch.Tensor, mag: float, q_out: torch.Tensor, kc: torch.Tensor | None,
+                    vc: torch.Tensor | None, q_weight: torch.Tensor | None = None, k_weight: torch.Tensor | None = None,
+                    eps: float = 0.0, conv_w: torch.Tensor | None = None, tails: torch.Tensor | None = None,
+                    half: bool = True):
+    """The step from an input projection to an attention layer's operands for layers that work on whole rows before the
+    heads are split, in one launch. q_in fp32 [T, H*dk], k_in [T, G*dk], v_in [T, G*dv] are column slices of one projection
+    output. In this order:
+      `conv_w` fp32 [taps, (H + G) dk] (query channels first, newest tap last): a causal convolution over time per channel,
+        no activation; each sequence's previous taps - 1 inputs are read from (and its newest written back to) `tails`
+        [slots, taps - 1, (H + G) dk] fp32, a chunk that starts at position 0 reads zeros;
+      `q_weight` / `k_weight` fp32 [H*dk] / [G*dk]: the whole row x / sqrt(mean(x^2) + eps) * weight;
+      rotation of the first 2 * len(freqs) numbers of every head, pairs (i, i + len(freqs)), or (2i, 2i + 1) without `half`,
+        by positions[t] * freqs[i]; sine and cosine times `mag`.
+    Queries go to q_out [T, H*dk], keys and values into the paged pools kc / vc at the rows' flat slots (< 0: not stored).
+    v_in = None: the values are the keys as they enter the rotation (dv = dk). k_in = None: queries only (a layer that reads
+    another layer's keys and values; convolution weights and tails then cover H dk channels)."""
+    T = q_in.shape[0]
+    if T == 0:
+        return
+    rot, C = 2 * freqs.numel(), (H + (G if k_in is not None else 0)) * dk
+    if rot > dk or freqs.dtype != torch.float32:
+        raise ValueError("row_rope_append: fp32 frequencies for at most the head's pairs")
+    if k_in is not None and v_in is None and dv != dk:
+        raise ValueError("row_rope_append: values that are keys have the keys' size")
+    if conv_w is not None:
+        taps = conv_w.shape[0]
+        if tuple(conv_w.shape) != (taps, C) or conv_w.dtype != torch.float32 or not conv_w.is_contiguous() or taps > 16:
+            raise ValueError("row_rope_append: convolution weights are fp32 [taps, channels], at most 16 taps")
+        if tails is None or tuple(tails.shape[1:]) != (max(1, taps - 1), C) or not tails.is_contiguous():
+            raise ValueError("row_rope_append: tails are [slots, taps - 1, channels]")
+    for w, n in ((q_weight, H * dk), (k_weight, G * dk)):
+        if w is not None and (w.dtype != torch.float32 or w.numel() != n or not w.is_contiguous()):
+            raise TypeError("row_rope_append: fp32 norm weights of one number per column")
+    if not q_in.is_cuda:
+        qk = q_in.float() if k_in is None else torch.cat([q_in.float(), k_in.float()], 1)
+        if conv_w is not None:
+            qk = causal_conv(qk, conv_w.t().contiguous(), None, tails, rag, torch.empty_like(qk), silu=False)
+
+        def turn(x, n, w):
+            if w is not None:
+                x = x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps) * w.float()
+            return x, _rope_ref(x.reshape(T, n, dk), rag.positions, rot, 1.0, half, freqs, mag).reshape(T, n * dk)
+        q_out.copy_(turn(qk[:, :H * dk], H, q_weight)[1])
+        if k_in is None:
+            return
+        flat, kr = turn(qk[:, H * dk:], G, k_weight)
+        ok = rag.slots >= 0
+        sl = rag.slots[ok].long()
+        kc.view(-1, G * dk)[sl] = kr[ok].to(kc.dtype)
+        vc.view(-1, G * dv)[sl] = (flat if v_in is None else v_in.float())[ok].to(vc.dtype)
+        return
+    for t_ in (q_in, k_in, v_in):
+        if t_ is not None:
+            _f32c(t_, "row_rope_append")
+    if k_in is not None and (kc.dtype != vc.dtype or kc.dtype != q_out.dtype or not kc.is_contiguous()
+                             or not vc.is_contiguous()):
+        raise TypeError("row_rope_append: queries and contiguous pools of one dtype")
+    ld = lambda t_: 0 if t_ is None else t_.stride(0)  # noqa: E731
+    i16 = _is16(q_out)
+    N.kcall("mxh_row_rope_append", q_in.data_ptr(), ld(q_in), N.ptr(k_in), ld(k_in), N.ptr(v_in), ld(v_in),
+            rag.positions.data_ptr(), rag.slots.data_ptr(), H, G, dk, dv, rot, int(half), freqs.data_ptr() if rot else None,
+            float(mag), N.ptr(q_weight), N.ptr(k_weight), float(eps), N.ptr(conv_w),
+            conv_w.shape[0] if conv_w is not None else 0, N.ptr(tails), rag.state.data_ptr(), rag.n_dec, N.ptr(rag.pf_cu),
+            rag.n_pf, q_out.data_ptr(), q_out.stride(0), i16, N.ptr(kc), N.ptr(vc), i16, T, N.stream_ptr())
+
+
 def _rope_ref(x: torch.Tensor, positions: torch.Tensor, rot_dims: int, rot_base: float, half: bool, freqs=None,
               mag: float = 1.0) -> torch.Tensor:
     """x fp32 [T, n, d]: a copy whose first rot_dims numbers per head are turned by the rows' positions."""
@@ -364,7 +436,7 @@ def rope_rows(x: torch.Tensor, positions: torch.Tensor, heads: int, dim: int, ro
 
 
 def _attn_ref(q, kc, vc, table, ctx, pos0, H, G, dk, dv, scale, chunk, window, sink, out, out_scale, sink_v=None,
-              bias=None, gate=None, Gv=None, keep=0):
+              bias=None, gate=None, Gv=None, keep=0, softcap=0.0):
     bs = kc.shape[1]
     nb = -(-ctx // bs)
     k = kc[table[:nb].long()].reshape(nb * bs, G, dk)[:ctx].float()
@@ -376,6 +448,8 @@ def _attn_ref(q, kc, vc, table, ctx, pos0, H, G, dk, dv, scale, chunk, window, s
     qh = q.float().reshape(n, H, dk)
     rep = H // G
     s = torch.einsum("nhd,jhd->hnj", qh, k.repeat_interleave(rep, 1)) * scale
+    if softcap:
+        s = softcap * torch.tanh(s / softcap)
     i = pos0 + torch.arange(n)[:, None]
     j = torch.arange(ctx)[None, :]
     lo = (i // chunk) * chunk if chunk else (i - window + 1).clamp(min=0) if window else torch.zeros_like(i)
@@ -391,7 +465,7 @@ def _attn_ref(q, kc, vc, table, ctx, pos0, H, G, dk, dv, scale, chunk, window, s
     den = e.sum(-1, keepdim=True) + (torch.exp(s0 - m) if sink else 0.0)
     o = torch.einsum("hnj,jhe->nhe", e / den, v.repeat_interleave(rep, 1))
     if gate is not None:
-        o = o * torch.sigmoid(gate.float())[:, :, None]
+        o = o * torch.sigmoid(gate.float()).reshape(n, H, -1)
     out.copy_((o.reshape(n, H * dv) * out_scale).to(out.dtype))
 
 
@@ -431,7 +505,7 @@ def _visible_blocks(p0: int, n: int, chunk: int, window: int, heads: int):
 
 
 def _attn_gemm_chunk(q, kc, vc, table, p0, n, H, G, dk, dv, scale, chunk, window, sink, out, out_scale, sink_v=None,
-                     bias=None, gate=None, Gv=None, p32=False, keep=0):
+                     bias=None, gate=None, Gv=None, p32=False, keep=0, softcap=0.0):
     """A long prompt chunk (rows q [n, H*dk] at positions p0 ..) as library GEMMs: per block of rows, the visible keys
     and values (with a window also the `keep` first tokens) are gathered head-major from the pages, scores = Q K^T
     (fp32), masked sink softmax, out = P V (fp32).
@@ -451,24 +525,26 @@ def _attn_gemm_chunk(q, kc, vc, table, p0, n, H, G, dk, dv, scale, chunk, window
         qh = torch.empty((H, n2, dk), dtype=md, device=dev)
         qr = q[a - p0:]
         N.kcall("mxh_head_transpose", qr.data_ptr(), i16, qr.stride(0), dk, qh.data_ptr(), i16, dk, n2 * dk, n2, H, dk,
-                1.0, None, 0, st)
+                1.0, None, 0, 1, st)
         sc = bmm_f32(qh.view(G, rep * n2, dk), kh.transpose(1, 2).contiguous())
         two = bool(p32 and i16)
         pw = torch.empty((G, rep * n2, 2 * nk if two else nk), dtype=md, device=dev)
         N.kcall("mxh_masked_softmax", sc.data_ptr(), pw.data_ptr(), i16, H * n2, n2, nk, a, key0, float(scale),
                 int(chunk), int(window), int(sink), N.ptr(sink_v), N.ptr(bias), bias.shape[1] if bias is not None else 0,
-                H, int(two), kn, int(keep), st)
+                H, int(two), kn, int(keep), float(softcap), st)
         o = bmm_f32(pw, torch.cat([vh, vh], 1) if two else vh)
         orow = out[a - p0:]
         grow = gate[a - p0:] if gate is not None else None
         N.kcall("mxh_head_transpose", o.data_ptr(), 0, dv, n2 * dv, orow.data_ptr(), _is16(out), orow.stride(0), dv, n2,
-                H, dv, float(out_scale), N.ptr(grow), grow.stride(0) if grow is not None else 0, st)
+                H, dv, float(out_scale), N.ptr(grow), grow.stride(0) if grow is not None else 0,
+                grow.shape[1] // H if grow is not None else 1, st)
 
 
 def masked_attention(q: torch.Tensor, kc: torch.Tensor, vc: torch.Tensor, rag: Ragged, H: int, G: int, dk: int, dv: int,
                      scale: float, out: torch.Tensor, chunk: int = 0, window: int = 0, sink=False,
                      out_scale: float = 1.0, workspace=None, bias: torch.Tensor | None = None,
-                     gate: torch.Tensor | None = None, v_heads: int | None = None, p32: bool = False, keep: int = 0):
+                     gate: torch.Tensor | None = None, v_heads: int | None = None, p32: bool = False, keep: int = 0,
+                     softcap: float = 0.0):
     """Causal attention of q [T, H*dk] over the paged pools (rope_norm_append's layout); query head h reads key
     head g = h // (H / G) and value head g % v_heads (v_heads = G when not given; fewer value heads than key heads:
     several attention maps over the same values). `p32`: softmax weights enter the value product with more than
@@ -478,13 +554,14 @@ def masked_attention(q: torch.Tensor, kc: torch.Tensor, vc: torch.Tensor, rag: R
     window the positions below `keep` stay visible as well, at their true distance. `sink` = True adds
     exp(0) to the softmax denominator, an fp32 tensor
     [H] adds exp(sink[h]). `bias` (fp32 [H, L], contiguous) adds bias[h, min(i - j, L - 1)] to the scaled score.
-    `gate` (fp32 [T, H], may be a column slice) multiplies head h's output of row t by sigmoid(gate[t, h]). out
-    [T, H*dv] (may be a column slice; fp32 or bf16) receives out_scale times the result. q, pools and out share fp32
+    `softcap` > 0 turns the scaled score s into softcap * tanh(s / softcap), before the bias and the mask.
+    `gate` (fp32 [T, H], may be a column slice) multiplies head h's output of row t by sigmoid(gate[t, h]); a gate of
+    [T, H*dv] numbers does so per value column. out [T, H*dv] (may be a column slice; fp32 or bf16) receives out_scale times the result. q, pools and out share fp32
     or bf16 operands; scores, softmax and the accumulators are fp32.
 
     On the GPU decode rows and short chunks run the row kernel (one wave per row and head; decode rows split their
     visible keys into partitions merged through `workspace` = (fp32 [rows, 2], fp32 [rows, dv]), rows >= n_dec * H
-    * partitions). bf16 tensors with head sizes of 64 or 128 run on the matrix cores: decode rows (up to 16 query
+    * partitions). bf16 tensors with head sizes of 64 or 128 (or 96 for both) run on the matrix cores: decode rows (up to 16 query
     heads per key head) and, when the step's chunk sizes are known on the host, chunks of MFMA_MIN_ROWS rows and more.
     Other chunks of GEMM_MIN_ROWS rows and more run as library GEMMs around a masked softmax kernel."""
     T = q.shape[0]
@@ -504,15 +581,18 @@ def masked_attention(q: torch.Tensor, kc: torch.Tensor, vc: torch.Tensor, rag: R
     if bias is not None and (bias.dtype != torch.float32 or bias.dim() != 2 or bias.shape[0] != H
                              or not bias.is_contiguous()):
         raise TypeError("masked_attention: the distance bias is a contiguous fp32 [H, distances] table")
-    if gate is not None and (gate.dtype != torch.float32 or gate.shape != (T, H) or gate.stride(1) != 1):
-        raise TypeError("masked_attention: the gate is fp32 [T, H]")
+    if gate is not None and (gate.dtype != torch.float32 or gate.shape not in ((T, H), (T, H * dv)) or gate.stride(1) != 1):
+        raise TypeError("masked_attention: the gate is fp32 [T, H] or [T, H * dv]")
+    if softcap < 0:
+        raise ValueError("masked_attention: the score cap is positive (0: none)")
     nd = rag.n_dec
     if not q.is_cuda:
         if nd:
             lens = rag.dec_lens.tolist()
             for i in range(nd):
                 _attn_ref(q[i:i + 1], kc, vc, rag.dec_bt[i], lens[i], lens[i] - 1, H, G, dk, dv, scale, chunk, window,
-                          sink, out[i:i + 1], out_scale, sink_v, bias, gate[i:i + 1] if gate is not None else None, Gv, keep)
+                          sink, out[i:i + 1], out_scale, sink_v, bias, gate[i:i + 1] if gate is not None else None, Gv, keep,
+                          softcap)
         if rag.n_pf:
             cu, ctx = rag.pf_cu.tolist(), rag.pf_ctx.tolist()
             for k in range(rag.n_pf):
@@ -521,7 +601,7 @@ def masked_attention(q: torch.Tensor, kc: torch.Tensor, vc: torch.Tensor, rag: R
                     r0 = nd + cu[k]
                     _attn_ref(q[r0:r0 + n], kc, vc, rag.pf_bt[k], ctx[k], ctx[k] - n, H, G, dk, dv, scale, chunk,
                               window, sink, out[r0:r0 + n], out_scale, sink_v, bias,
-                              gate[r0:r0 + n] if gate is not None else None, Gv, keep)
+                              gate[r0:r0 + n] if gate is not None else None, Gv, keep, softcap)
         return out
     if q.dtype != kc.dtype or kc.dtype != vc.dtype or q.stride(1) != 1 or out.stride(1) != 1:
         raise TypeError("masked_attention: queries and pools share one dtype, rows are contiguous")
@@ -530,6 +610,8 @@ def masked_attention(q: torch.Tensor, kc: torch.Tensor, vc: torch.Tensor, rag: R
     common = (H, G, dk, dv, float(scale), int(chunk), int(window), int(sink), float(out_scale))
     nb = bias.shape[1] if bias is not None else 0
     ldg = gate.stride(0) if gate is not None else 0
+    gw = gate.shape[1] // H if gate is not None else 1
+    cap = float(softcap)
     extra = (N.ptr(sink_v), N.ptr(bias), nb)  # the gate pointer moves with the rows a launch serves
     mfma_ok = q.dtype == torch.bfloat16 and q.stride(0) % 8 == 0 and MFMA_MIN_ROWS > 0 and \
         bool(N.hybrid_kernels().mxh_attention_mfma_ok(dk, dv))
@@ -551,12 +633,12 @@ def masked_attention(q: torch.Tensor, kc: torch.Tensor, vc: torch.Tensor, rag: R
                     rag.dec_bt.data_ptr(), rag.dec_bt.stride(0), rag.dec_lens.data_ptr(), nd, out.data_ptr(),
                     out.stride(0), _is16(out), H, G, dk, dv, float(scale), int(chunk), int(window), int(sink),
                     float(out_scale), parts, plen if parts > 1 else 0, N.ptr(ml), N.ptr(po), *extra, N.ptr(gate), ldg,
-                    Gv, int(p32), int(keep), st)
+                    Gv, int(p32), int(keep), gw, cap, st)
         else:
             N.kcall("mxh_attention", q.data_ptr(), q.stride(0), _is16(q), kc.data_ptr(), vc.data_ptr(), bs,
                     rag.dec_bt.data_ptr(), rag.dec_bt.stride(0), None, rag.dec_lens.data_ptr(), nd, nd, 0,
                     out.data_ptr(), out.stride(0), _is16(out), *common, 0, parts, plen if parts > 1 else 0, N.ptr(ml),
-                    N.ptr(po), *extra, N.ptr(gate), ldg, Gv, int(keep), st)
+                    N.ptr(po), *extra, N.ptr(gate), ldg, Gv, int(keep), gw, cap, st)
     if rag.n_pf:
         lens = rag.pf_q_host if len(rag.pf_q_host) == rag.n_pf and len(rag.pf_ctx_host) == rag.n_pf else None
 
@@ -564,7 +646,7 @@ def masked_attention(q: torch.Tensor, kc: torch.Tensor, vc: torch.Tensor, rag: R
             N.kcall("mxh_attention", q.data_ptr(), q.stride(0), _is16(q), kc.data_ptr(), vc.data_ptr(), bs,
                     rag.pf_bt.data_ptr(), rag.pf_bt.stride(0), rag.pf_cu.data_ptr(), rag.pf_ctx.data_ptr(), rag.n_pf,
                     n_rows, nd, out.data_ptr(), out.stride(0), _is16(out), *common, row_off, 1, 0, None, None, *extra,
-                    N.ptr(gate), ldg, Gv, int(keep), st)
+                    N.ptr(gate), ldg, Gv, int(keep), gw, cap, st)
         mfma = mfma_ok
         big = MFMA_MIN_ROWS if mfma else GEMM_MIN_ROWS
         if lens is None or max(lens) < big or (not mfma and 0 < chunk < GEMM_MIN_ROWS):
@@ -582,10 +664,10 @@ def masked_attention(q: torch.Tensor, kc: torch.Tensor, vc: torch.Tensor, rag: R
                     N.kcall("mxh_attention_mfma", qk.data_ptr(), qk.stride(0), kc.data_ptr(), vc.data_ptr(), bs,
                             rag.pf_bt[k].data_ptr(), rag.pf_ctx_host[k] - n, n, ok.data_ptr(), ok.stride(0), _is16(out),
                             H, G, dk, dv, float(scale), int(chunk), int(window), int(sink), float(out_scale), *extra,
-                            N.ptr(gk), ldg, Gv, int(p32), int(keep), st)
+                            N.ptr(gk), ldg, Gv, int(p32), int(keep), gw, cap, st)
                 else:
                     _attn_gemm_chunk(qk, kc, vc, rag.pf_bt[k], rag.pf_ctx_host[k] - n, n, H, G, dk, dv, scale, chunk,
-                                     window, sink, ok, out_scale, sink_v, bias, gk, Gv, p32, keep)
+                                     window, sink, ok, out_scale, sink_v, bias, gk, Gv, p32, keep, softcap)
             elif n and run0 is None:
                 run0 = r
             r += n
@@ -634,6 +716,47 @@ def causal_conv(x: torch.Tensor, w: torch.Tensor, bias: torch.Tensor | None, tai
 
 
 # ------------------------------------------------------------------------------------------------ recurrences
+def mlstm_gates(zi: torch.Tensor, zf: torch.Tensor, bias_i: torch.Tensor | None, bias_f: torch.Tensor | None, cap: float,
+                peak: torch.Tensor, rag: Ragged, decay: torch.Tensor, coef: torch.Tensor, floor: torch.Tensor):
+    """Exponential gates of a matrix memory, per token and head in the order of each sequence's rows:
+        i = cap tanh((zi + bias_i) / cap);  f = log sigmoid(cap tanh((zf + bias_f) / cap));  m <- max(f + m_before, i)
+        decay = exp(f + m_before - m);  coef = exp(i - m);  floor = exp(-m)
+    The running maximum m starts at 0 and is carried in `peak` (fp32 [slots, H]); a chunk that starts at position 0 ignores
+    what its slot held. zi, zf fp32 [T, H] (column slices of one projection output); decay, coef, floor fp32 [T, H]
+    contiguous. With S <- decay S + coef k v^T and n alike, S and n are the memory divided by exp(m), and exp(-m) is what a
+    bound of 1 on |n . q| becomes."""
+    T, H = zi.shape
+    if T == 0:
+        return
+    if cap <= 0:
+        raise ValueError("mlstm_gates: the gates' cap is positive")
+    if not zi.is_cuda:
+        i = cap * torch.tanh((zi.float() if bias_i is None else zi.float() + bias_i) / cap)
+        f = F.logsigmoid(cap * torch.tanh((zf.float() if bias_f is None else zf.float() + bias_f) / cap))
+        st, pos = rag.state.tolist(), rag.positions.tolist()
+        for r0, n, si in rag.host_segments():
+            slot = st[si]
+            m = torch.zeros(H) if (pos[r0] == 0 or slot < 0) else peak[slot].clone()
+            for t in range(r0, r0 + n):
+                new = torch.maximum(f[t] + m, i[t])
+                decay[t], coef[t], floor[t], m = torch.exp(f[t] + m - new), torch.exp(i[t] - new), torch.exp(-new), new
+            if slot >= 0:
+                peak[slot] = m
+        return
+    if zi.stride(0) != zf.stride(0):
+        raise ValueError("mlstm_gates: both gates are columns of one projection output")
+    for v in (zi, zf):
+        _f32c(v, "mlstm_gates")
+    for v in (decay, coef, floor):
+        if v.dtype != torch.float32 or v.shape != (T, H) or not v.is_contiguous():
+            raise TypeError("mlstm_gates: contiguous fp32 [T, H] outputs")
+    if peak.dtype != torch.float32 or peak.shape[1] != H or not peak.is_contiguous():
+        raise TypeError("mlstm_gates: the carried maximum is fp32 [slots, H]")
+    N.kcall("mxh_mlstm_gates", zi.data_ptr(), zf.data_ptr(), zi.stride(0), N.ptr(bias_i), N.ptr(bias_f), float(cap),
+            peak.data_ptr(), rag.state.data_ptr(), rag.positions.data_ptr(), rag.n_dec, N.ptr(rag.pf_cu), rag.n_pf,
+            decay.data_ptr(), coef.data_ptr(), floor.data_ptr(), H, N.stream_ptr())
+
+
 def unit_norm_heads(x: torch.Tensor, heads: int, dim: int, eps: float, scale: float = 1.0, split: int | None = None,
                     scale2: float = 1.0):
     """In place on fp32 x [T, heads*dim]: every head becomes x / sqrt(sum(x^2) + eps) * scale; heads from index
@@ -707,7 +830,8 @@ def channel_decay(z: torch.Tensor, bias: torch.Tensor | None, tau: float, out: t
 
 def state_scan(k: torch.Tensor, q: torch.Tensor, v: torch.Tensor, decay: torch.Tensor, coef: torch.Tensor | None,
                skip: torch.Tensor | None, state: torch.Tensor, rag: Ragged, out: torch.Tensor, H: int, G: int, Nk: int,
-               P: int, delta: bool, channel: bool = False, q_scale: float = 1.0, coef_sigmoid: bool = False):
+               P: int, delta: bool, channel: bool = False, q_scale: float = 1.0, coef_sigmoid: bool = False,
+               norm_out: torch.Tensor | None = None):
     """Linear recurrence per sequence and head over the step's rows, in order:
         S <- decay_t S;  u = coef_t (v_t - S^T k_t) if delta else coef_t v_t;  S <- S + k_t u^T;
         o_t = S^T (q_scale q_t) (+ skip_h v_t)
@@ -716,7 +840,8 @@ def state_scan(k: torch.Tensor, q: torch.Tensor, v: torch.Tensor, decay: torch.T
     channel (row n of S is multiplied by decay[h, n]: gated linear attention, or with `delta` a delta rule with a decay
     per key channel). A decay of shape [H] is one constant per head for every token (retention). coef = None means 1;
     with `coef_sigmoid` coef holds pre-activations (a column slice of a projection's output) and the write strength is
-    their sigmoid.
+    their sigmoid. `norm_out` (fp32 [T, H], contiguous): the state has one more column per head, [slots, H, P + 1, Nk],
+    which holds n <- decay n + coef k (a value of 1 at every token), and norm_out receives n^T (q_scale q).
     state fp32 [slots, H, P, Nk] (a column's Nk numbers are contiguous) is read at
     the sequence's slot unless its first row is at position 0 (then S starts at zero) and written back after its last
     row."""
@@ -726,13 +851,16 @@ def state_scan(k: torch.Tensor, q: torch.Tensor, v: torch.Tensor, decay: torch.T
     if not k.is_cuda:
         st, pos = rag.state.tolist(), rag.positions.tolist()
         rep = H // G
+        Pn = P + (norm_out is not None)
         for r0, n, si in rag.host_segments():
             slot = st[si]
-            S = torch.zeros(H, Nk, P) if (pos[r0] == 0 or slot < 0) else state[slot].transpose(1, 2).clone()
+            S = torch.zeros(H, Nk, Pn) if (pos[r0] == 0 or slot < 0) else state[slot].transpose(1, 2).clone()
             for t in range(r0, r0 + n):
                 kt = k[t].float().reshape(G, Nk).repeat_interleave(rep, 0)
                 qt = q[t].float().reshape(G, Nk).repeat_interleave(rep, 0) * q_scale
                 vt = v[t].float().reshape(H, P)
+                if norm_out is not None:
+                    vt = torch.cat([vt, torch.ones(H, 1)], 1)
                 dt = decay if decay.dim() == 1 else decay[t]
                 S = S * (dt.reshape(H, Nk)[:, :, None] if channel else dt[:, None, None])
                 cf = 1.0
@@ -743,13 +871,19 @@ def state_scan(k: torch.Tensor, q: torch.Tensor, v: torch.Tensor, decay: torch.T
                 o = torch.einsum("hnp,hn->hp", S, qt)
                 if skip is not None:
                     o = o + skip[:, None] * vt
-                out[t] = o.reshape(H * P)
+                out[t] = o[:, :P].reshape(H * P)
+                if norm_out is not None:
+                    norm_out[t] = o[:, P]
             if slot >= 0:
                 state[slot] = S.transpose(1, 2)
         return out
     for t_ in (k, q, v, out):
         _f32c(t_, "state_scan")
-    if tuple(state.shape[1:]) != (H, P, Nk) or not state.is_contiguous() or not decay.is_contiguous() \
+    Pn = P + (norm_out is not None)
+    if norm_out is not None and (norm_out.shape != (T, H) or norm_out.dtype != torch.float32
+                                 or not norm_out.is_contiguous()):
+        raise TypeError("state_scan: the normaliser's output is a contiguous fp32 [T, H]")
+    if tuple(state.shape[1:]) != (H, Pn, Nk) or not state.is_contiguous() or not decay.is_contiguous() \
             or (coef is not None and (coef.stride(1) != 1 or coef.dtype != torch.float32)) or H % G or Nk > 256:
         raise ValueError("state_scan: state is [slots, H, P, N] with N <= 256, decay contiguous, coef fp32 [T, H]")
     if decay.shape[-1] != (H * Nk if channel else H) or (decay.dim() == 1 and channel) or decay.dtype != torch.float32:
@@ -759,18 +893,20 @@ def state_scan(k: torch.Tensor, q: torch.Tensor, v: torch.Tensor, decay: torch.T
             coef.stride(0) if coef is not None else 0, int(coef_sigmoid), N.ptr(skip), state.data_ptr(),
             rag.state.data_ptr(),
             rag.positions.data_ptr(), rag.n_dec, N.ptr(rag.pf_cu), rag.n_pf, out.data_ptr(), out.stride(0), H, G, Nk,
-            P, int(delta), int(channel), float(q_scale), N.stream_ptr())
+            P, int(delta), int(channel), float(q_scale), N.ptr(norm_out), N.stream_ptr())
     return out
 
 
 def gated_group_norm(y: torch.Tensor, gate: torch.Tensor, w: torch.Tensor | None, eps: float, group: int,
                      out: torch.Tensor, gate_first: bool, out_scale: float = 1.0, act: str = "silu",
-                     proj: torch.Tensor | None = None):
+                     proj: torch.Tensor | None = None, den: torch.Tensor | None = None,
+                     den_min: torch.Tensor | None = None, den_eps: float = 0.0):
     """Rows y [T, C] fp32 in groups of `group` columns, gate [T, C] fp32 (pre-activation), w fp32 whose length divides
     C (column c uses w[c % len(w)]; None: no weight). gate_first: z = y * act(gate), out = unit_rms_group(z) * w;
     otherwise out = unit_rms_group(y) * w * act(gate); act is "silu" or "sigmoid". With `proj` (fp32 [R, C], contiguous)
     the gate is [T, R] and its pre-activation is gate proj, summed in fp32 inside the kernel (the second half of a
-    low-rank gate). out (fp32 or bf16, may be a column slice) gets out_scale times that."""
+    low-rank gate). With `den` and `den_min` (fp32 [T, C / group], contiguous) every group of y is first divided by
+    max(|den|, den_min) + den_eps. out (fp32 or bf16, may be a column slice) gets out_scale times that."""
     T, C = y.shape
     if T == 0:
         return out
@@ -782,7 +918,13 @@ def gated_group_norm(y: torch.Tensor, gate: torch.Tensor, w: torch.Tensor | None
         raise ValueError("gated_group_norm: group size and weight length divide the row")
     if gate.shape != ((T, proj.shape[0]) if proj is not None else (T, C)) or (proj is not None and proj.shape[1] != C):
         raise ValueError("gated_group_norm: the gate is [T, C], or [T, R] beside a projection [R, C]")
+    if (den is None) != (den_min is None) or (den is not None and (
+            den.shape != (T, C // group) or den_min.shape != den.shape or den.dtype != torch.float32
+            or den_min.dtype != torch.float32 or not den.is_contiguous() or not den_min.is_contiguous())):
+        raise ValueError("gated_group_norm: one fp32 divisor and one bound per row and group")
     if not y.is_cuda:
+        if den is not None:
+            y = y / (torch.maximum(den.abs(), den_min) + den_eps).repeat_interleave(group, 1)
         gp = gate.float() @ proj.float() if proj is not None else gate.float()
         g = F.silu(gp) if act == "silu" else torch.sigmoid(gp)
         z = (y.float() * g if gate_first else y.float()).reshape(T, C // group, group)
@@ -795,7 +937,8 @@ def gated_group_norm(y: torch.Tensor, gate: torch.Tensor, w: torch.Tensor | None
         raise TypeError("gated_group_norm: the projection is a contiguous fp32 [R, C] matrix")
     N.kcall("mxh_gated_group_norm", y.data_ptr(), y.stride(0), gate.data_ptr(), gate.stride(0), w.data_ptr(),
             w.numel(), float(eps), group, int(gate_first), float(out_scale), out.data_ptr(), out.stride(0), _is16(out),
-            T, C, int(act == "sigmoid"), N.ptr(proj), proj.shape[0] if proj is not None else 0, N.stream_ptr())
+            T, C, int(act == "sigmoid"), N.ptr(proj), proj.shape[0] if proj is not None else 0, N.ptr(den),
+            N.ptr(den_min), C // group, float(den_eps), N.stream_ptr())
     return out
 
 
@@ -835,7 +978,8 @@ def diff_group_norm(a: torch.Tensor, b: torch.Tensor, lam: float, eps: float, gr
 
 
 # ------------------------------------------------------------------------------------------------ feed-forward
-GLU_ACTS = {"silu": 0, "gelu_tanh": 1, "relu2": 2, "clamped": 3}
+GLU_ACTS = {"silu": 0, "gelu_tanh": 1, "relu2": 2, "clamped": 3, "gelu": 4}
+GLU_SINGLE = ("relu2", "gelu")  # units without a second operand
 
 
 def glu(a: torch.Tensor, b: torch.Tensor | None, bias_a: torch.Tensor | None, bias_b: torch.Tensor | None,
@@ -847,12 +991,13 @@ def glu(a: torch.Tensor, b: torch.Tensor | None, bias_a: torch.Tensor | None, bi
     sigmoid first with `scale_sigmoid`. act "relu2" has no second operand (b = None) and the factor multiplies the
     INPUT: out = relu(factor * (a + bias_a))^2, an expert that is fed its routing weight times the token.
     act "clamped": out = g sigmoid(alpha g) (u + 1) [* factor] with g = min(a + bias_a, limit) and
-    u = clamp(b + bias_b, -limit, limit)."""
+    u = clamp(b + bias_b, -limit, limit). act "gelu" has no second operand either: out = gelu(a + bias_a) [* factor], the
+    exact form with erf."""
     T, Fn = a.shape
     if T == 0 or Fn == 0:
         return out
-    if act not in GLU_ACTS or (b is None) != (act == "relu2"):
-        raise ValueError("glu: act is silu | gelu_tanh | clamped with two operands, or relu2 with one")
+    if act not in GLU_ACTS or (b is None) != (act in GLU_SINGLE):
+        raise ValueError("glu: act is silu | gelu_tanh | clamped with two operands, or relu2 | gelu with one")
     if not a.is_cuda:
         x = a.float() + bias_a if bias_a is not None else a.float()
         s = None
@@ -861,6 +1006,8 @@ def glu(a: torch.Tensor, b: torch.Tensor | None, bias_a: torch.Tensor | None, bi
             s = s.repeat_interleave(group, 1)
         if act == "relu2":
             z = torch.relu(x * s if s is not None else x).pow(2)
+        elif act == "gelu":
+            z = F.gelu(x) if s is None else F.gelu(x) * s
         else:
             y = b.float() + bias_b if bias_b is not None else b.float()
             if act == "clamped":
