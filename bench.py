@@ -96,13 +96,13 @@ def parse():
                     help="comma list of sampling phases measured back to back on the same server: reference = "
                          "the reference's defaults (temperature 0.9, top_k 40, top_p 0.95; backend_config.go "
                          "SetDefaults) on the GPU sampler; greedy = argmax. The first phase is the headline")
-    ap.add_argument("--arch-bench", default="", choices=["", "vosotar", "vugotar", "girulorn", "keronex", "zomolix"],
+    ap.add_argument("--arch-bench", default="", choices=["", "vosotar", "vugotar", "girulorn", "keronex", "zomolix", "tebodra"],
                     help="instead of the headline serving benchmark: prefill and decode throughput of this model "
                          "family beside the Llama graph at equal layer sizes (random bf16 / f16 weights, one GPU)")
     ap.add_argument("--arch-sizes", default="1b,7b", help="--arch-bench: comma list of layer sizes (1b, 7b)")
     ap.add_argument("--arch-layers", type=int, default=4, help="--arch-bench: layers per model")
     ap.add_argument("--arch-models", default="", help="--arch-bench: comma list to restrict the models (vosotar, vugotar, girulorn, "
-                         "keronex, zomolix, vugotar-moe, llama-f16)")
+                         "keronex, zomolix, tebodra, vugotar-moe, llama-f16)")
     ap.add_argument("--arch-batches", default="1,32", help="--arch-bench: decode batch sizes")
     ap.add_argument("--arch-chunk", type=int, default=2048, help="--arch-bench vugotar: attention chunk size")
     return ap.parse_args()
@@ -311,6 +311,36 @@ def run_arch_bench(args) -> int:
                                 g_heads=s["heads"] // 2, g_dim=128, g_vdim=128, tau=12.0, rank=32, name=f"girulorn-{sz}",
                                 **moe)
             yield "girulorn", lambda: GI.GirulornModel.load(gc, GI.synthetic_source(gc, 1), dev, torch.bfloat16)
+        elif args.arch_bench == "tebodra":
+            # a chunked attention layer, one that borrows its keys, a matrix memory and an attention layer whose values are
+            # its keys in turn; attention heads as the Llama graph's (GQA 4:1, head size 128), chunks as long as Vugotar's, half
+            # as many memory heads with 128 x 128 states; dense feed-forwards of two matrices, 1.5 times as wide so that
+            # they hold as many weights as the gated ones. Beside it the framework's two closest models: Vugotar (chunked
+            # sink attention beside a delta rule with a short convolution, a state-space layer every fourth, dense
+            # feed-forward) and Keronex on a single residual with dense feed-forwards (differential attention, retention: a
+            # plain scan of the same states).
+            from localai_tfp_amd.models import keronex as KE
+            from localai_tfp_amd.models import tebodra as TE
+            from localai_tfp_amd.models import vugotar as VU
+            kinds = ("attention_2", "attention_2", "mlstm", "attention")
+            kv = max(1, s["heads"] // 4)
+            tc = TE.make_config(hidden=s["hidden"], vocab=V, pattern=tuple(kinds[i % 4] for i in range(nl)),
+                                kv_from={i: i - 1 for i in range(1, nl, 4)}, heads=s["heads"], kv_heads=kv, dim=128, vdim=128,
+                                chunk=args.arch_chunk, rot_base=5e5, rot_factor=4.0, t_rot_dims=64, t_rot_base=5e5,
+                                t_scaling=(8.0, 1.0, 4.0, 8192.0), conv=4, softcap=50.0, m_heads=s["heads"] // 2, m_dim=128,
+                                m_vdim=128, gate_cap=15.0, ff=s["ff"] * 3 // 2, residual_mult=0.3, name=f"tebodra-{sz}")
+            yield "tebodra", lambda: TE.TebodraModel.load(tc, TE.synthetic_source(tc, 1), dev, torch.bfloat16)
+            uc = VU.make_config(hidden=s["hidden"], vocab=V, pattern=tuple("mamba2" if i % 4 == 3 else "parallel" for i in range(nl)),
+                                mlps=("dense",), heads=s["heads"], kv_heads=kv, dim=128, vdim=128, chunk=args.arch_chunk,
+                                d_heads=s["heads"] // 2, d_kv_heads=kv, d_dim=128, d_vdim=128, d_conv=4,
+                                m_heads=2 * s["hidden"] // 64, m_vdim=64, m_state=128, m_groups=1, m_norm_groups=1, m_conv=4,
+                                ff=s["ff"], name=f"vugotar-{sz}")
+            yield "vugotar", lambda: VU.VugotarModel.load(uc, VU.synthetic_source(uc, 1), dev, torch.bfloat16)
+            kc = KE.make_config(hidden=s["hidden"], vocab=V,
+                                pattern=tuple("retention" if i % 4 == 2 else "attention" for i in range(nl)), heads=s["heads"],
+                                kv_heads=kv, dim=64, vdim=128, rot_dims=64, r_heads=s["heads"] // 2, r_dim=128, r_vdim=128,
+                                mlps=("dense",), ff=s["ff"], streams=None, bigram=None, name=f"keronex-{sz}")
+            yield "keronex", lambda: KE.KeronexModel.load(kc, KE.synthetic_source(kc, 1), dev, torch.bfloat16)
         elif args.arch_bench == "vugotar":
             # attention + delta-rule layers with a state-space layer every fourth, dense feed-forwards; attention
             # heads as the Llama graph's (GQA 4:1, head size 128), delta rule with half as many heads of 128 x 128

@@ -102,17 +102,21 @@ def gated_output(o, h, get, p):
     return (o * torch.sigmoid(h @ get(p + "g").to(F64).T)) @ get(p + "o").to(F64).T
 
 
-def tied_mixer(m, get, p, h):
-    """Attention whose values are its keys as the convolution leaves them."""
+def tied_mixer(m, get, p, h, kv_of):
+    """Attention whose values are its keys as the convolution leaves them. `kv_of`: layer index -> (keys as they are scored,
+    values) of the attention layers run so far."""
     T, H, G, d = h.shape[0], m["heads"], m["kv_heads"], m["dim"]
     q = short_conv(h @ get(p + "q").to(F64).T, get(p + "q.conv")).reshape(T, H, d)
-    k = short_conv(h @ get(p + "k").to(F64).T, get(p + "k.conv")).reshape(T, G, d)
-    o = grouped_attention(rotate(q, m.get("rot")), rotate(k, m.get("rot")), k, m["scale"], m.get("softcap"))
-    return gated_output(o.reshape(T, H * d), h, get, p)
+    if m.get("kv_from") is None:
+        v = short_conv(h @ get(p + "k").to(F64).T, get(p + "k.conv")).reshape(T, G, d)
+        k = rotate(v, m.get("rot"))
+    else:
+        k, v = kv_of[m["kv_from"]]
+    o = grouped_attention(rotate(q, m.get("rot")), k, v, m["scale"], m.get("softcap"))
+    return gated_output(o.reshape(T, H * d), h, get, p), (k, v)
 
 
 def chunked_mixer(m, get, p, h, eps, kv_of):
-    """`kv_of`: layer index -> (normed, rotated keys, values) of the chunked layers run so far."""
     T, H, G, d, e = h.shape[0], m["heads"], m["kv_heads"], m["dim"], m["vdim"]
     q = rotate(plain_norm(h @ get(p + "q").to(F64).T, get(p + "q.norm"), eps).reshape(T, H, d), m.get("rot"))
     if m.get("kv_from") is None:
@@ -180,7 +184,7 @@ def forward(d, get, tokens, layers=None):
         p = f"l{i}.mix."
         h = offset_norm(x, get(f"l{i}.norm1"), eps)
         if L["type"] == "attention":
-            y = tied_mixer(L["mixer"], get, p, h)
+            y, kv[i] = tied_mixer(L["mixer"], get, p, h, kv)
         elif L["type"] == "attention_2":
             y, kv[i] = chunked_mixer(L["mixer"], get, p, h, eps, kv)
         else:
