@@ -4,11 +4,14 @@
 // heads; rotary positions; the queries as a GEMM-side operand and keys and values into the paged pools. Without a value
 // projection the values are the keys as they enter the rotation.
 //
-// One block per (token, part): part 0 the query heads, part 1 the key heads, part 2 the value heads. A thread owns
-// ITEMS of its row: a rotation pair, or one number outside the rotated part, so a pair's two numbers never leave the
-// thread and the row needs no LDS. Rows of up to blockDim.x * RK items wait in registers between the statistics and the
-// rotation; longer ones are read again. Sine and cosine are computed once per (token, pair) and shared by all heads
-// through LDS. Everything is fp32 up to the stores.
+// A block serves one token and one part: some or all of its query items, of its key items, or its value heads. An ITEM is a
+// rotation pair, or one number outside the rotated part: a pair's two numbers stay in one thread and the row needs no LDS.
+// With whole-row norms a part is a whole row (up to blockDim.x * RK items wait in registers between the statistics and the
+// rotation, longer rows are read again); without them it is blockDim.x * RK items, so that a single token spreads over
+// several CUs. All taps' inputs of all items are requested together (a tap before the chunk's first row points into the
+// carried inputs, one before the sequence's start into anything and is dropped), and a single new token rolls its
+// channels' carried inputs from those same registers. Sine and cosine are computed once per block and pair and shared by
+// the heads through LDS. Everything is fp32 up to the stores.
 #include "../mx_common.h"
 
 namespace {
@@ -40,26 +43,27 @@ struct RowRope {
     void *kc, *vc;
 };
 
-// TAPS: 0 no convolution, else the loop bound (a.taps <= TAPS)
+// TAPS: 1 without a convolution, else the bound of the tap loops (a.taps <= TAPS). grid (T, bq + bk + values)
 template <bool Q16, bool C16, int TAPS, int RK>
-__global__ __launch_bounds__(1024) void row_rope_append_kernel(RowRope a) {
+__global__ __launch_bounds__(1024) void row_rope_append_kernel(RowRope a, int bq, int bk) {
     extern __shared__ float trig[];  // [rot / 2] cosines, [rot / 2] sines
     __shared__ float red[16];
-    const int t = blockIdx.x, part = blockIdx.y, nt = blockDim.x, tid = threadIdx.x;
-    const long slot = part ? a.slots[t] : 0;
-    if (part == 2) {
+    const int t = blockIdx.x, nt = blockDim.x, tid = threadIdx.x;
+    const bool isq = (int)blockIdx.y < bq;
+    const long slot = isq ? 0 : a.slots[t];
+    if ((int)blockIdx.y >= bq + bk) {
         if (slot < 0) return;
         const float* src = a.v + (long)t * a.ldv;
         const int n = a.G * a.dv;
         for (int c = tid; c < n; c += nt) st_elem<C16>(a.vc, slot * n + c, src[c]);
         return;
     }
-    const bool isq = part == 0;
+    const int part = isq ? blockIdx.y : blockIdx.y - bq, parts = isq ? bq : bk;
     const int heads = isq ? a.H : a.G;
     const int n2 = a.rot >> 1, per = a.dk - n2;  // items per head: n2 pairs, then the unrotated numbers
     const int n_items = heads * per;
     const int ld = isq ? a.ldq : a.ldk;
-    const float* src = isq ? a.q : a.k;
+    const float* src = (isq ? a.q : a.k) + (long)t * ld;
     const float* w = isq ? a.qw : a.kw;
     const int ch0 = isq ? 0 : a.H * a.dk;  // first convolution channel of the part
     const float pos = (float)a.positions[t];
@@ -69,12 +73,13 @@ __global__ __launch_bounds__(1024) void row_rope_append_kernel(RowRope a) {
         trig[i] = c * a.mag;
         trig[n2 + i] = s * a.mag;
     }
-    // the row's place in its sequence's chunk
-    int since = 0;  // rows of the chunk before this one
-    float* tail = nullptr;  // the sequence's carried inputs (null: it starts at position 0, or carries nothing)
-    bool roll = false;  // a single new token rolls its own channels' carried inputs
-    if constexpr (TAPS > 0) {
-        int s;
+    const float* in[TAPS];  // the part's inputs b rows back
+    bool live[TAPS];        // false: before the sequence's start
+    float* roll = nullptr;  // a single new token's carried inputs
+    in[0] = src;
+    live[0] = true;
+    if constexpr (TAPS > 1) {
+        int s, since = 0;  // the row's sequence, rows of its chunk before it
         if (t < a.n_dec) {
             s = t;
         } else {
@@ -88,40 +93,16 @@ __global__ __launch_bounds__(1024) void row_rope_append_kernel(RowRope a) {
             since = t - a.n_dec - a.pf_cu[lo];
         }
         const int sl = a.state[s];
-        if (sl >= 0 && a.taps > 1) {
-            float* p = a.tails + (long)sl * (a.taps - 1) * a.C + ch0;
-            if (a.positions[t - since] != 0) tail = p;
-            roll = t < a.n_dec;
+        float* tail = a.tails + (long)max(sl, 0) * (a.taps - 1) * a.C + ch0;
+        const bool carried = sl >= 0 && a.positions[t - since] != 0;
+        if (sl >= 0 && t < a.n_dec && a.taps > 1) roll = tail;
+#pragma unroll
+        for (int b = 1; b < TAPS; ++b) {
+            const bool tap = b < a.taps, here = b <= since;
+            live[b] = tap && (here || carried);
+            in[b] = !live[b] ? src : here ? src - (long)b * ld : tail + (long)(a.taps - 1 - b + since) * a.C;
         }
     }
-    // the number at channel e of the part's row: the projection, or its convolution
-    auto value = [&](int e) {
-        if constexpr (TAPS == 0) {
-            return src[(long)t * ld + e];
-        } else {
-            float x[TAPS], acc = 0.f;
-#pragma unroll
-            for (int b = 0; b < TAPS; ++b) {  // b rows back
-                x[b] = 0.f;
-                if (b < a.taps) {
-                    if (b <= since) x[b] = src[(long)(t - b) * ld + e];
-                    else if (tail) x[b] = tail[(long)(a.taps - 1 - b + since) * a.C + e];
-                }
-            }
-#pragma unroll
-            for (int b = TAPS - 1; b >= 0; --b)
-                if (b < a.taps) acc += a.cw[(long)(a.taps - 1 - b) * a.C + ch0 + e] * x[b];
-            return acc;
-        }
-    };
-    auto roll_tail = [&](int e) {
-        if constexpr (TAPS > 0) {
-            float* p = a.tails + (long)a.state[t] * (a.taps - 1) * a.C + ch0 + e;
-            for (int i = 0; i + 2 < a.taps; ++i) p[(long)i * a.C] = tail ? p[(long)(i + 1) * a.C] : 0.f;
-            p[(long)(a.taps - 2) * a.C] = src[(long)t * ld + e];
-        }
-    };
-    float x0[RK], x1[RK];
     auto locate = [&](int it, int& e0, int& e1, int& u) {
         const int hd = it / per;
         u = it - hd * per;
@@ -129,39 +110,89 @@ __global__ __launch_bounds__(1024) void row_rope_append_kernel(RowRope a) {
         e0 = hd * a.dk + (pair ? (a.half ? u : 2 * u) : u + n2);
         e1 = pair ? (a.half ? e0 + n2 : e0 + 1) : e0;
     };
-    auto load = [&](int base) {
-        float ss = 0.f;
+    float x0[RK], x1[RK];
+    // the items from `base` on, into x0 / x1; returns the thread's sum of squares
+    auto load = [&](int base, bool last) {
+        float r0[RK][TAPS], r1[RK][TAPS];
 #pragma unroll
         for (int r = 0; r < RK; ++r) {
-            const int it = base + tid + r * nt;
             int e0, e1, u;
-            locate(min(it, n_items - 1), e0, e1, u);  // clamped: straight-line loads, all in flight together
-            x0[r] = value(e0);
-            x1[r] = value(e1);
-            if (it < n_items) ss += x0[r] * x0[r] + (u < n2 ? x1[r] * x1[r] : 0.f);
+            locate(min(base + tid + r * nt, n_items - 1), e0, e1, u);  // clamped: straight-line loads, all in flight together
+#pragma unroll
+            for (int b = 0; b < TAPS; ++b) {
+                r0[r][b] = in[b][e0];
+                r1[r][b] = in[b][e1];
+            }
         }
-        return ss;
+        if constexpr (TAPS > 1) {
+            float ss = 0.f;
+#pragma unroll
+            for (int r = 0; r < RK; ++r) {
+                int e0, e1, u;
+                locate(min(base + tid + r * nt, n_items - 1), e0, e1, u);
+                x0[r] = x1[r] = 0.f;
+#pragma unroll
+                for (int b = TAPS - 1; b >= 0; --b) {
+                    const float* cw = a.cw + (long)max(a.taps - 1 - b, 0) * a.C + ch0;
+                    const float w0 = cw[e0], w1 = cw[e1];
+                    x0[r] += w0 * (live[b] ? r0[r][b] : 0.f);
+                    x1[r] += w1 * (live[b] ? r1[r][b] : 0.f);
+                }
+                if (base + tid + r * nt < n_items) ss += x0[r] * x0[r] + (u < n2 ? x1[r] * x1[r] : 0.f);
+            }
+            if (last && roll) {
+#pragma unroll
+                for (int r = 0; r < RK; ++r) {
+                    const int it = base + tid + r * nt;
+                    int e0, e1, u;
+                    locate(min(it, n_items - 1), e0, e1, u);
+                    if (it < n_items) {
+#pragma unroll
+                        for (int b = 0; b < TAPS - 1; ++b) {
+                            if (b < a.taps - 1) {
+                                roll[(long)(a.taps - 2 - b) * a.C + e0] = live[b] ? r0[r][b] : 0.f;
+                                if (u < n2) roll[(long)(a.taps - 2 - b) * a.C + e1] = live[b] ? r1[r][b] : 0.f;
+                            }
+                        }
+                    }
+                }
+            }
+            return ss;
+        } else {
+            float ss = 0.f;
+#pragma unroll
+            for (int r = 0; r < RK; ++r) {
+                const int it = base + tid + r * nt;
+                x0[r] = r0[r][0];
+                x1[r] = r1[r][0];
+                if (it < n_items) ss += x0[r] * x0[r] + (it % per < n2 ? x1[r] * x1[r] : 0.f);
+            }
+            return ss;
+        }
     };
-    const bool cached = n_items <= nt * RK;
+    const int stride = nt * RK;
+    const bool cached = w && n_items <= stride;
     float sc = 1.f;
-    float ss = 0.f;
-    if (cached) ss = load(0);
-    else if (w)
-        for (int base = 0; base < n_items; base += nt * RK) ss += load(base);
     if (w) {
+        float ss = 0.f;
+        if (cached) ss = load(0, true);
+        else
+            for (int base = 0; base < n_items; base += stride) ss += load(base, false);
         ss = wave_sum(ss);
         if ((tid & 63) == 0) red[tid >> 6] = ss;
+    } else {
+        load(part * stride, true);  // requested before the wait for the angles
     }
     __syncthreads();  // the statistics and the angles
     if (w) {
-        ss = 0.f;
+        float ss = 0.f;
         for (int i = 0; i < nt >> 6; ++i) ss += red[i];
         sc = 1.f / sqrtf(ss / (float)(heads * a.dk) + a.eps);
     }
     const bool tied = !isq && !a.v;
     const long row_q = (long)t * a.ldqo, row_c = slot * (long)(a.G * a.dk);
-    for (int base = 0; base < n_items; base += nt * RK) {
-        if (!cached) load(base);
+    for (int base = part * stride; base < n_items; base += parts * stride) {
+        if (w ? !cached : base != part * stride) load(base, true);
 #pragma unroll
         for (int r = 0; r < RK; ++r) {
             const int it = base + tid + r * nt;
@@ -190,10 +221,6 @@ __global__ __launch_bounds__(1024) void row_rope_append_kernel(RowRope a) {
                     st_elem<C16>(a.vc, row_c + e0, y0);
                     if (pair) st_elem<C16>(a.vc, row_c + e1, y1);
                 }
-            }
-            if (roll) {
-                roll_tail(e0);
-                if (pair) roll_tail(e1);
             }
         }
     }
@@ -240,21 +267,30 @@ extern "C" int mxh_row_rope_append(const float* q, int ldq, const float* k, int 
     RowRope a = {q,  k,  v,   ldq, ldk, ldv,  positions, slots, H, g, dk, dv, rot, half, freqs, mag,
                  qw, kw, eps, cw,  cw ? taps : 0, (H + g) * dk, tails, state, n_dec, pf_cu, n_pf, qo, ldqo, kc, vc};
     constexpr int RK = 4;
-    const int items = max(H, g) * (dk - rot / 2);
-    const int nt = items <= 1024 ? 256 : 1024;
-    const dim3 grid(T, k ? (v ? 3 : 2) : 1);
+    const int per = dk - rot / 2, items = max(H, g) * per;
+    // whole rows for the norms, else 512 items (two per thread) to a block
+    const int nt = qw && items > 1024 ? 1024 : 256;
+    const int bq = qw ? 1 : (H * per + 511) / 512, bk = !k ? 0 : kw ? 1 : (g * per + 511) / 512;
+    MXH_CHECK(bq + bk < 65535);
+    const dim3 grid(T, bq + bk + (v ? 1 : 0));
     const size_t sh = rot * sizeof(float);
-#define GO2(Q, C_, TP) row_rope_append_kernel<Q, C_, TP, RK><<<grid, nt, sh, st>>>(a)
+#define GO2(Q, C_, TP, R_) row_rope_append_kernel<Q, C_, TP, R_><<<grid, nt, sh, st>>>(a, bq, bk)
+#define GO1(Q, C_, TP)             \
+    do {                           \
+        if (qw) GO2(Q, C_, TP, RK); \
+        else GO2(Q, C_, TP, 2);    \
+    } while (0)
 #define GO(Q, C_)                        \
     do {                                 \
-        if (!cw) GO2(Q, C_, 0);          \
-        else if (taps <= 4) GO2(Q, C_, 4); \
-        else GO2(Q, C_, 16);             \
+        if (!cw) GO1(Q, C_, 1);          \
+        else if (taps <= 4) GO1(Q, C_, 4); \
+        else GO2(Q, C_, 16, 2);          \
     } while (0)
     if (q16 && c16) GO(true, true);
     else if (!q16 && !c16) GO(false, false);
     else return (int)hipErrorInvalidValue;
 #undef GO
+#undef GO1
 #undef GO2
     if (cw && taps > 1 && n_pf > 0)
         row_tails_kernel<<<dim3((a.C + 255) / 256, n_pf), 256, 0, st>>>(a, H * dk);

@@ -228,12 +228,12 @@ __global__ __launch_bounds__(256) void state_scan_kernel(const float* k, int ldk
 // blockDim.x tokens at a time (a wave-wide prefix, the waves' totals through LDS), and every token reads its
 // predecessor's m as that one computed it, so stored states and scales always refer to the same number. m starts at 0
 // and is carried in peak[slot][h]. grid (H, sequences)
-__global__ __launch_bounds__(256) void mlstm_gates_kernel(const float* zi, const float* zf, int ldz, const float* bi,
+__global__ __launch_bounds__(1024) void mlstm_gates_kernel(const float* zi, const float* zf, int ldz, const float* bi,
                                                           const float* bf, float cap, float* peak, const int* seq_state,
                                                           const int* positions, int n_dec, const int* pf_cu,
                                                           float* decay, float* coef, float* floor_, int H) {
-    __shared__ float ms[257];  // m of the token before the round's first, then of its tokens
-    __shared__ float ta[4], tb[4];  // a wave's 64 maps composed
+    __shared__ float ms[1025];  // m of the token before the round's first, then of its tokens
+    __shared__ float ta[16], tb[16];  // a wave's 64 maps composed
     const int h = blockIdx.x, s = blockIdx.y, nt = blockDim.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     int row0, n;
     if (s < n_dec) {
@@ -331,12 +331,13 @@ extern "C" int mxh_state_scan(const float* k, int ldk, const float* q, int ldq, 
 
 extern "C" int mxh_mlstm_gates(const float* zi, const float* zf, int ldz, const float* bi, const float* bf, float cap,
                                float* peak, const int* seq_state, const int* positions, int n_dec, const int* pf_cu,
-                               int n_pf, float* decay, float* coef, float* floor_, int H, hipStream_t st) {
+                               int n_pf, float* decay, float* coef, float* floor_, int H, int T, hipStream_t st) {
     const int n_seqs = n_dec + n_pf;
     if (n_seqs <= 0) return 0;
     MXH_CHECK(zi && zf && peak && seq_state && positions && decay && coef && floor_ && (n_pf == 0 || pf_cu));
     MXH_CHECK(H > 0 && ldz >= H && cap > 0.f && n_seqs <= 65535);
-    mlstm_gates_kernel<<<dim3(H, n_seqs), n_pf ? 256 : 64, 0, st>>>(zi, zf, ldz, bi, bf, cap, peak, seq_state, positions,
-                                                                    n_dec, pf_cu, decay, coef, floor_, H);
+    const int nt = n_pf ? min(1024, (max(T - n_dec, 1) + 63) / 64 * 64) : 64;  // a prompt chunk of up to 1024 rows in one round
+    mlstm_gates_kernel<<<dim3(H, n_seqs), nt, 0, st>>>(zi, zf, ldz, bi, bf, cap, peak, seq_state, positions, n_dec, pf_cu,
+                                                       decay, coef, floor_, H);
     return (int)hipGetLastError();
 }

@@ -157,8 +157,8 @@ HYBRID_SIGS = {
     # taps, tails, seq_state, n_dec, pf_cu, n_pf, q_out, ldqo, q16, kc, vc, c16, T, stream
     "mxh_row_rope_append": [P, I, P, I, P, I, P, P, I, I, I, I, I, I, P, F, P, P, F, P, I, P, P, I, P, I, P, I, I, P, P, I,
                             I, P],
-    # zi, zf, ldz, bias_i, bias_f, cap, peak, seq_state, positions, n_dec, pf_cu, n_pf, decay, coef, floor, H, stream
-    "mxh_mlstm_gates": [P, P, I, P, P, F, P, P, P, I, P, I, P, P, P, I, P],
+    # zi, zf, ldz, bias_i, bias_f, cap, peak, seq_state, positions, n_dec, pf_cu, n_pf, decay, coef, floor, H, T, stream
+    "mxh_mlstm_gates": [P, P, I, P, P, F, P, P, P, I, P, I, P, P, P, I, I, P],
     # q, k, v, ldq, ldk, ldv, positions, H, G, dk, dv, rot_dims, base, norm, eps, q_out, ldqo, q16, kc, vc, c16, slots,
     # q_weight, k_weight, temp_coef, temp_every, T, stream
     # ..., temp_every, half, value heads, freqs, mag, q_bias, k_bias, v_bias, T, stream

@@ -505,7 +505,7 @@ class TebodraModel:
                            kv[0] if own else None, kv[1] if own else None, W.q_norm, W.k_norm, eps, W.conv_w, tails)
         HY.masked_attention(q, kv[0], kv[1], rag, H, G, dk, dv, a.scale, cat[:, :H * dv], chunk=a.chunk,
                             sink=False if a.tied else W.sink, softcap=a.softcap, gate=col("g", H * dv),
-                            workspace=(ws.part_ml, ws.part_o))
+                            workspace=(ws.part_ml, ws.part_o), p32=True)
 
     def _mlstm(self, r: MlstmCfg, W, y, rag, state, peak, ws, cat, eps):
         T = y.shape[0]

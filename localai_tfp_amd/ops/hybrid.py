@@ -754,7 +754,7 @@ def mlstm_gates(zi: torch.Tensor, zf: torch.Tensor, bias_i: torch.Tensor | None,
         raise TypeError("mlstm_gates: the carried maximum is fp32 [slots, H]")
     N.kcall("mxh_mlstm_gates", zi.data_ptr(), zf.data_ptr(), zi.stride(0), N.ptr(bias_i), N.ptr(bias_f), float(cap),
             peak.data_ptr(), rag.state.data_ptr(), rag.positions.data_ptr(), rag.n_dec, N.ptr(rag.pf_cu), rag.n_pf,
-            decay.data_ptr(), coef.data_ptr(), floor.data_ptr(), H, N.stream_ptr())
+            decay.data_ptr(), coef.data_ptr(), floor.data_ptr(), H, T, N.stream_ptr())
 
 
 def unit_norm_heads(x: torch.Tensor, heads: int, dim: int, eps: float, scale: float = 1.0, split: int | None = None,
