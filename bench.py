@@ -326,9 +326,9 @@ def run_arch_bench(args) -> int:
             kv = max(1, s["heads"] // 4)
             tc = TE.make_config(hidden=s["hidden"], vocab=V, pattern=tuple(kinds[i % 4] for i in range(nl)),
                                 kv_from={i: i - 1 for i in range(1, nl, 4)}, heads=s["heads"], kv_heads=kv, dim=128, vdim=128,
-                                chunk=args.arch_chunk, rot_base=5e5, rot_factor=4.0, t_rot_dims=64, t_rot_base=5e5,
+                                chunk=args.arch_chunk, rot_base=1e5, rot_factor=2.0, t_rot_dims=64, t_rot_base=1e5,
                                 t_scaling=(8.0, 1.0, 4.0, 8192.0), conv=4, softcap=50.0, m_heads=s["heads"] // 2, m_dim=128,
-                                m_vdim=128, gate_cap=15.0, ff=s["ff"] * 3 // 2, residual_mult=0.3, name=f"tebodra-{sz}")
+                                m_vdim=128, gate_cap=15.0, ff=s["ff"] * 3 // 2, residual_mult=0.25, name=f"tebodra-{sz}")
             yield "tebodra", lambda: TE.TebodraModel.load(tc, TE.synthetic_source(tc, 1), dev, torch.bfloat16)
             uc = VU.make_config(hidden=s["hidden"], vocab=V, pattern=tuple("mamba2" if i % 4 == 3 else "parallel" for i in range(nl)),
                                 mlps=("dense",), heads=s["heads"], kv_heads=kv, dim=128, vdim=128, chunk=args.arch_chunk,

@@ -4,8 +4,8 @@
 // The value pool may hold fewer heads than the key pool (gv of them, a divisor of G): key head g then reads value head
 // g % gv, several attention maps over the same values. Every kernel also takes an AttnExtra: a learned sink score per
 // head instead of 0, an additive bias looked up by the distance between query and key (table [H, distances], the last
-// entry serving every larger distance), a gate per row and head (or per row, head and value column) whose sigmoid multiplies the
-// output, a cap of the scores, and a count of first tokens (`keep`) that stay visible in front of a window.
+// entry serving every larger distance), a gate per row and head (or per row, head and value column) whose sigmoid
+// multiplies the output, a cap of the scores, and a count of first tokens (`keep`) that stay visible in front of a window.
 //
 // attn_rows_kernel: one wave per (query row, query head). Keys are taken 64 at a time, one per lane: the lane forms
 // its key's whole score against the query (held in LDS as fp32, pre-multiplied by the scale), the wave updates the
@@ -15,8 +15,8 @@
 // With parts > 1 (decode rows of long contexts) grid.z splits a row's visible keys into partitions whose
 // (max, sum, unnormalised output) go to a workspace; attn_merge_kernel combines them in a fixed order and adds the sink.
 //
-// bf16 pools with head sizes of 64 / 128 (or 96 for both) run on the matrix cores instead: attn_chunk_mfma_kernel for prompt chunks,
-// attn_decode_mfma_kernel for single new tokens (both further down, with their fragment layouts).
+// bf16 pools with head sizes of 64 / 128 (or 96 for both) run on the matrix cores instead: attn_chunk_mfma_kernel for
+// prompt chunks, attn_decode_mfma_kernel for single new tokens (both further down, with their fragment layouts).
 //
 // Other long prompt chunks take another route (ops/hybrid.py): kv_gather_kernel copies the chunk's visible keys and values
 // from the pages into head-major matrices, head_transpose_kernel does the same for the queries, the library computes
@@ -535,7 +535,7 @@ __global__ __launch_bounds__(256) void attn_chunk_mfma_kernel(const bf16_t* __re
     }
 }
 
-// attn_decode_mfma_kernel: single new tokens on the matrix cores (bf16 pools, head sizes 64 / 128, up to 16 query heads
+// attn_decode_mfma_kernel: single new tokens on the matrix cores (bf16 pools, head sizes as above, up to 16 query heads
 // per key / value head). grid (sequences, G, partitions), one wave per workgroup: the 16 rows of its tile are the
 // query heads that share key / value head blockIdx.y (rows beyond H / G are zero), all at the sequence's newest
 // position, so a key and value tile is read once for all of them. The wave walks its partition's keys

@@ -117,7 +117,7 @@ __global__ __launch_bounds__(1024) void row_rope_append_kernel(RowRope a, int bq
 #pragma unroll
         for (int r = 0; r < RK; ++r) {
             int e0, e1, u;
-            locate(min(base + tid + r * nt, n_items - 1), e0, e1, u);  // clamped: straight-line loads, all in flight together
+            locate(min(base + tid + r * nt, n_items - 1), e0, e1, u);  // clamped: no branch between the loads
 #pragma unroll
             for (int b = 0; b < TAPS; ++b) {
                 r0[r][b] = in[b][e0];
@@ -226,8 +226,8 @@ __global__ __launch_bounds__(1024) void row_rope_append_kernel(RowRope a, int bq
     }
 }
 
-// grid (ceil(C / 256), chunks), launched after the rows: a chunk's newest taps - 1 inputs become the sequence's carried ones.
-// Channels 0 .. nq - 1 come from q, the others from k. Single new tokens have rolled theirs.
+// grid (ceil(C / 256), chunks), launched after the rows: a chunk's newest taps - 1 inputs become the sequence's carried
+// ones. Channels 0 .. nq - 1 come from q, the others from k. Single new tokens have rolled theirs.
 __global__ __launch_bounds__(256) void row_tails_kernel(RowRope a, int nq) {
     const int c = blockIdx.x * 256 + threadIdx.x, k = blockIdx.y, nt = a.taps - 1;
     const int row0 = a.n_dec + a.pf_cu[k], n = a.pf_cu[k + 1] - a.pf_cu[k], slot = a.state[a.n_dec + k];

@@ -165,8 +165,8 @@ def _state_families():
 def _load_latent(model: str, device, tp_size: int, ov: dict):
     """Latent-attention decoders (models/vosotar.py, models/zomolix.py) and hybrid attention / recurrent decoders
     (models/vugotar.py, models/girulorn.py, models/keronex.py, models/tebodra.py): a directory whose config.json names the
-    architecture, or `synthetic:<family>-*` random weights. `overrides["dtype"]`: torch.bfloat16 (default on GPU) | torch.float32. None
-    for everything else."""
+    architecture, or `synthetic:<family>-*` random weights. `overrides["dtype"]`: torch.bfloat16 (default on GPU) |
+    torch.float32. None for everything else."""
     from ..tokenizer import ByteTokenizer
     fam = None
     for key, (mod, klass, is_dir) in _state_families().items():

@@ -217,7 +217,7 @@ class TebodraConfig:
 def make_config(hidden=128, vocab=320, pattern=("attention_2", "mlstm", "attention"), heads=4, kv_heads=2, dim=32, vdim=32,
                 scale=None, chunk=48, rot_dims=None, rot_base=10000.0, rot_factor=None, kv_from=None, t_heads=None,
                 t_kv_heads=None, t_dim=None, t_scale=None, t_rot_dims=None, t_rot_base=10000.0, t_scaling=None, conv=4,
-                softcap=30.0, m_heads=4, m_dim=32, m_vdim=32, gate_cap=15.0, mlps=("dense",), ff=256, residual_mult=0.5,
+                softcap=50.0, m_heads=4, m_dim=32, m_vdim=32, gate_cap=15.0, mlps=("dense",), ff=256, residual_mult=0.5,
                 eps=1e-6, name="tebodra") -> TebodraConfig:
     """A configuration whose i-th layer has mixer pattern[i] and feed-forward mlps[i % len(mlps)] ("dense" | None).
     heads .. rot_factor describe the chunked layers (`chunk` may be a map from the layer index, `rot_factor` is a linear
@@ -252,12 +252,12 @@ SYNTHETIC = {
     "tebodra-tiny": dict(hidden=144, vocab=352, pattern=("attention_2", "mlstm", "attention", "attention_2"), kv_from={3: 0},
                          mlps=("dense", None)),
     "tebodra-1b": dict(hidden=2048, vocab=32000, pattern=_PAT * 4, kv_from={i: i - 1 for i in range(1, 16, 4)}, heads=16,
-                       kv_heads=4, dim=128, vdim=128, chunk=2048, rot_factor=4.0, rot_base=5e5, t_rot_dims=64,
-                       t_rot_base=5e5, t_scaling=(8.0, 1.0, 4.0, 8192.0), softcap=50.0, m_heads=8, m_dim=128, m_vdim=256,
+                       kv_heads=4, dim=128, vdim=128, chunk=2048, rot_factor=2.0, rot_base=1e5, t_rot_dims=64,
+                       t_rot_base=1e5, t_scaling=(8.0, 1.0, 4.0, 8192.0), softcap=50.0, m_heads=8, m_dim=128, m_vdim=256,
                        ff=8192, residual_mult=0.25),
     "tebodra-7b": dict(hidden=4096, vocab=32000, pattern=_PAT * 8, kv_from={i: i - 1 for i in range(1, 32, 4)}, heads=32,
-                       kv_heads=8, dim=128, vdim=128, chunk=2048, rot_factor=4.0, rot_base=5e5, t_rot_dims=64,
-                       t_rot_base=5e5, t_scaling=(8.0, 1.0, 4.0, 8192.0), softcap=50.0, m_heads=16, m_dim=128, m_vdim=256,
+                       kv_heads=8, dim=128, vdim=128, chunk=2048, rot_factor=2.0, rot_base=1e5, t_rot_dims=64,
+                       t_rot_base=1e5, t_scaling=(8.0, 1.0, 4.0, 8192.0), softcap=50.0, m_heads=16, m_dim=128, m_vdim=256,
                        ff=14336, residual_mult=0.18),
 }
 

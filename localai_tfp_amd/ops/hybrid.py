@@ -469,7 +469,7 @@ def _attn_ref(q, kc, vc, table, ctx, pos0, H, G, dk, dv, scale, chunk, window, s
     out.copy_((o.reshape(n, H * dv) * out_scale).to(out.dtype))
 
 
-MFMA_MIN_ROWS = 16  # bf16 prompt chunks of at least this many rows take the matrix-core kernel (head sizes 64 / 128)
+MFMA_MIN_ROWS = 16  # bf16 prompt chunks of at least this many rows take the matrix-core kernel (head sizes 64 / 96 / 128)
 GEMM_MIN_ROWS = 64  # other prompt chunks of at least this many rows take the library-GEMM route (GPU)
 GEMM_MAX_SCORES = 1 << 26  # fp32 scores of one sub-problem of that route
 DECODE_WAVES = 4096  # decode rows: waves to aim for when splitting contexts into key partitions
@@ -556,13 +556,13 @@ def masked_attention(q: torch.Tensor, kc: torch.Tensor, vc: torch.Tensor, rag: R
     [H] adds exp(sink[h]). `bias` (fp32 [H, L], contiguous) adds bias[h, min(i - j, L - 1)] to the scaled score.
     `softcap` > 0 turns the scaled score s into softcap * tanh(s / softcap), before the bias and the mask.
     `gate` (fp32 [T, H], may be a column slice) multiplies head h's output of row t by sigmoid(gate[t, h]); a gate of
-    [T, H*dv] numbers does so per value column. out [T, H*dv] (may be a column slice; fp32 or bf16) receives out_scale times the result. q, pools and out share fp32
-    or bf16 operands; scores, softmax and the accumulators are fp32.
+    [T, H*dv] numbers does so per value column. out [T, H*dv] (may be a column slice; fp32 or bf16) receives out_scale
+    times the result. q, pools and out share fp32 or bf16 operands; scores, softmax and the accumulators are fp32.
 
     On the GPU decode rows and short chunks run the row kernel (one wave per row and head; decode rows split their
     visible keys into partitions merged through `workspace` = (fp32 [rows, 2], fp32 [rows, dv]), rows >= n_dec * H
-    * partitions). bf16 tensors with head sizes of 64 or 128 (or 96 for both) run on the matrix cores: decode rows (up to 16 query
-    heads per key head) and, when the step's chunk sizes are known on the host, chunks of MFMA_MIN_ROWS rows and more.
+    * partitions). bf16 tensors with head sizes of 64 or 128 (or 96 for both) run on the matrix cores: decode rows (up
+    to 16 query heads per key head) and, when the step's chunk sizes are known on the host, chunks of MFMA_MIN_ROWS rows and more.
     Other chunks of GEMM_MIN_ROWS rows and more run as library GEMMs around a masked softmax kernel."""
     T = q.shape[0]
     if T == 0:

@@ -29,7 +29,7 @@ DEVS = ["cpu", GPU]
 RUNS = [("cpu", "float32", 2e-4), pytest.param("cuda", "float32", 2e-4, marks=pytest.mark.gpu),
         pytest.param("cuda", "bfloat16", 6e-2, marks=pytest.mark.gpu)]
 F64 = torch.float64
-BANDS = (4.0, 1.0, 4.0, 60.0)  # (factor, low, high, original): kept, blended and divided pairs among these small heads'
+BANDS = (3.0, 1.0, 5.0, 60.0)  # (factor, low, high, original): kept, blended and divided pairs among these small heads'
 
 SHAPES = {
     # all mixers, a layer that borrows keys under a chunk of its own, both kinds of scaled rotation, a layer without a
@@ -48,8 +48,8 @@ SHAPES = {
     # numbers per column, one memory head, no feed-forward anywhere
     "wide": dict(hidden=48, vocab=53, pattern=("mlstm", "attention", "attention_2", "attention_2"), kv_from={3: 2}, heads=4,
                  kv_heads=1, dim=72, vdim=8, chunk={2: 33, 3: 50}, rot_dims=0, scale=0.2, t_heads=5, t_kv_heads=1, t_dim=40,
-                 t_rot_dims=10, t_scaling=(8.0, 0.5, 2.0, 40.0), conv=7, softcap=30.0, m_heads=1, m_dim=160, m_vdim=72,
-                 gate_cap=3.0, mlps=(None,), residual_mult=0.3),
+                 t_rot_dims=10, t_scaling=(8.0, 0.5, 2.0, 40.0), conv=7, softcap=25.0, m_heads=1, m_dim=160, m_vdim=72,
+                 gate_cap=3.0, mlps=(None,), residual_mult=0.4),
     # nothing a multiple of eight, one tap, no cap, chunks of one token, plain causal among the "chunked" ones
     "ragged": dict(hidden=44, vocab=101, pattern=("attention_2", "attention", "attention_2", "mlstm"), heads=5, kv_heads=5,
                    dim=20, vdim=12, chunk={0: 1, 2: 0}, rot_dims=10, rot_factor=7.0, scale=0.3, t_heads=3, t_kv_heads=1,
@@ -101,8 +101,8 @@ def test_frequencies_with_and_without_scaling():
         assert TE.RotCfg.from_json(TE.RotCfg.from_json(rot).to_json()) == TE.RotCfg.from_json(rot)
     plain = O.frequencies({"dims": 24, "base": 700.0})
     banded = O.frequencies({"dims": 24, "base": 700.0, "scaling": bands})
-    assert banded[0] == plain[0] and banded[-1] == plain[-1] / 4.0  # short waves kept, long ones divided, a blend between
-    assert ((banded < plain) & (banded > plain / 4.0)).sum() > 0
+    assert banded[0] == plain[0] and banded[-1] == plain[-1] / 3.0  # short waves kept, long ones divided, a blend between
+    assert ((banded < plain) & (banded > plain / 3.0)).sum() > 0
     assert TE.RotCfg().table("cpu").numel() == 0
 
 
